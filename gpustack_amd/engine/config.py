@@ -122,7 +122,20 @@ class PagedMixerSpec:
       with one learned l per layer; the blend is what the pool keeps.
     * softcap > 0: the scaled score s becomes softcap * tanh(s / softcap).
     * head_norm together with a rotation (rot.dims > 0) and biases: the
-      per-head norm comes first, then the rotation."""
+      per-head norm comes first, then the rotation.
+    * chunk > 0: a row sees the keys of its own chunk of positions only,
+      floor(j / chunk) == floor(i / chunk), chunks counted from the start of
+      the sequence.
+    * unit_sink: a sink whose score is the constant 0 (one more in the
+      softmax denominator), nothing learned.
+    * unit_norm: every q and k head is divided by its root mean square, no
+      weight (a rotation keeps a head's length, so this and the rotation
+      may come in either order).
+    * conv > 0: q, k and v pass a causal convolution of `conv` taps per
+      channel (no bias, no activation) right after the projection; the last
+      conv - 1 projected rows are kept in the sequence's state slot.
+    * out_gate: each head's output times a sigmoid gate read from the
+      mixer's input."""
     heads: int
     kv_heads: int
     qk_dim: int
@@ -142,6 +155,11 @@ class PagedMixerSpec:
     distance_bias: bool = False
     v_mix: bool = False
     softcap: float = 0.0
+    chunk: int = 0
+    unit_sink: bool = False
+    unit_norm: bool = False
+    conv: int = 0
+    out_gate: bool = False
 
     def slopes(self) -> list[float]:
         """Distance-bias slope of every head, in double precision."""
@@ -155,6 +173,13 @@ class PagedMixerSpec:
     @property
     def v_width(self) -> int:
         return self.qk_dim if self.tied_values else self.v_dim
+
+    @property
+    def conv_channels(self) -> int:     # q | k | v
+        if not self.conv:
+            return 0
+        return (self.maps * self.qk_dim * (self.heads + self.kv_heads)
+                + (0 if self.tied_values else self.kv_heads * self.v_dim))
 
 
 @dataclass(frozen=True)
@@ -195,6 +220,16 @@ class ScanMixerSpec:
     @property
     def conv_channels(self) -> int:     # x | B | C
         return (self.inner + 2 * self.groups * self.state) if self.conv else 0
+
+
+@dataclass(frozen=True)
+class GruMixerSpec:
+    """Gated recurrence with one fp32 state value per channel and sequence
+    (models/state_mixers.py MinGruMixer), S_t = (1 - z_t) S_(t-1) + z_t c_t,
+    whose gate z = sigmoid(.) and candidate c (u + 1/2 for u >= 0, else
+    sigmoid(u)) are read from the current token only; the state, times a
+    SiLU gate, goes through the output projection."""
+    width: int
 
 
 @dataclass(frozen=True)
@@ -240,9 +275,10 @@ class FeedForwardSpec:
 @dataclass(frozen=True)
 class LayerSpec:
     """One entry of a heterogeneous layer stack (ModelSpec.layers)."""
-    # "latent_attention" | "paged_attention" | "scan" | "parallel"
+    # "latent_attention" | "paged_attention" | "scan" | "parallel" | "gru"
     mixer_type: str
-    mixer: "LatentMixerSpec | PagedMixerSpec | ScanMixerSpec | ParallelMixerSpec"
+    mixer: ("LatentMixerSpec | PagedMixerSpec | ScanMixerSpec"
+            " | ParallelMixerSpec | GruMixerSpec")
     mlp: FeedForwardSpec | None = None
 
 
@@ -369,6 +405,15 @@ class ModelSpec:
     layer_loop: tuple | None = None      # (start, stop, times)
     # the embedding output passes a norm of its own before the first layer
     embed_norm: bool = False
+    # hyper-connections (models/hyper_streams.py): the residual is `streams`
+    # parallel fp32 streams with learned input, mixing and output weights
+    # per sublayer. 0 = one plain residual stream
+    streams: int = 0
+    # a mixer reads h + (h_prev - h) * shift, h_prev the normed row of the
+    # previous token, which the sequence's state slot carries between steps
+    token_shift: bool = False
+    # every sublayer's result is multiplied by sigmoid(W h + b), h its input
+    residual_gate: bool = False
 
     @property
     def gqa_ratio(self) -> int:
@@ -406,7 +451,7 @@ class ModelSpec:
                     out.append(("kv", 1, m.kv_rank + m.rot_dim, m.kv_rank))
                 else:
                     out.append(("latent", m.kv_rank))
-            elif isinstance(m, ScanMixerSpec):
+            elif isinstance(m, (ScanMixerSpec, GruMixerSpec)):
                 out.append(("state",))      # nothing per token: a state slot
             else:
                 out.append(("kv", m.kv_heads, m.k_width, m.v_width))
@@ -414,7 +459,8 @@ class ModelSpec:
 
     def state_pool_shapes(self) -> list[tuple | None]:
         """Per layer run: None, or (heads, state, vdim, conv rows, conv
-        channels) of the recurrent state one live sequence holds there."""
+        channels) of the recurrent state one live sequence holds there
+        (heads 0: convolution rows only)."""
         out = []
         for i, _ in self.layer_runs():
             m = self.layers[i].mixer
@@ -423,24 +469,31 @@ class ModelSpec:
             if isinstance(m, ScanMixerSpec):
                 out.append((m.heads, m.state, m.vdim,
                             max(m.conv - 1, 0), m.conv_channels))
+            elif isinstance(m, GruMixerSpec):
+                out.append((1, 1, m.width, 0, 0))
+            elif isinstance(m, PagedMixerSpec) and m.conv:
+                out.append((0, 0, 0, m.conv - 1, m.conv_channels))
             else:
                 out.append(None)
         return out
 
     def state_bytes_per_slot(self, dtype_size: int = 2) -> int:
         """Bytes one live sequence holds in the recurrent-state pool: fp32
-        matrix states plus the convolutions' last inputs in the engine
-        dtype, over all layer runs."""
+        states plus the convolutions' last inputs and the token shift's
+        previous rows in the engine dtype, over all layer runs."""
         if self.layers is None:
             return 0
-        return sum(sh[0] * sh[1] * sh[2] * 4 + sh[3] * sh[4] * dtype_size
-                   for sh in self.state_pool_shapes() if sh is not None)
+        n = sum(sh[0] * sh[1] * sh[2] * 4 + sh[3] * sh[4] * dtype_size
+                for sh in self.state_pool_shapes() if sh is not None)
+        if self.token_shift:
+            n += len(self.layer_runs()) * self.hidden_size * dtype_size
+        return n
 
     @property
     def has_state(self) -> bool:
-        return self.layers is not None and any(
-            isinstance(ls.mixer, (ScanMixerSpec, ParallelMixerSpec))
-            for ls in self.layers)
+        return self.layers is not None and (
+            self.token_shift
+            or any(sh is not None for sh in self.state_pool_shapes()))
 
     def kv_bytes_per_token(self, dtype_size: int = 2) -> int:
         if self.layers is not None:
@@ -463,6 +516,9 @@ class ModelSpec:
                 n += (self.bigram_buckets + 1) * h
             for ls in self.layers:
                 m = ls.mixer
+                if self.streams:
+                    n += self._stream_layer_weights(h, ls)
+                    continue
                 if self.architecture == "Makezen":
                     n += self._mixer_weights(h, m) + 2 * h
                     if ls.mlp is not None:
@@ -558,6 +614,21 @@ class ModelSpec:
              + 2 * m.heads + m.heads * h + m.heads * m.v_dim * h)
         if m.kv_from < 0:
             n += h * (m.kv_rank + m.rot_dim) + m.kv_rank
+        return n
+
+    def _stream_layer_weights(self, h: int, ls) -> int:
+        """Weight count of one layer on parallel residual streams."""
+        m, f, s = ls.mixer, ls.mlp, self.streams
+        sub = s * s + 2 * s + h + (h * h + h if self.residual_gate else 0)
+        n = sub + (h if self.token_shift else 0)
+        if isinstance(m, GruMixerSpec):
+            n += 4 * h * m.width + 2 * m.width
+        else:
+            qkv = (m.qk_dim * (m.heads + m.kv_heads) + m.kv_heads * m.v_dim)
+            n += (h * qkv + qkv * m.conv + m.heads * m.v_dim * h
+                  + (m.heads * h if m.out_gate else 0))
+        if f is not None:
+            n += sub + (3 if f.gated else 2) * h * f.ff
         return n
 
     @staticmethod
@@ -910,7 +981,82 @@ class ModelSpec:
         )
 
     @classmethod
+    def _from_fuvuvik_config(cls, cfg: dict) -> "ModelSpec":
+        """Fuvuvik checkpoints list their layers one by one; an entry names
+        its mixer — "attention" (short convolution on q, k and v, rotation,
+        unit q / k heads, plain causal softmax), "attention_2" (rotation,
+        keys of the row's own chunk, one more in the denominator) or
+        "mingru" (gated recurrence) — and a gated dense feed-forward or
+        none. The residual is `streams` parallel fp32 streams, every mixer
+        input is shifted towards the previous token's, every sublayer's
+        result is gated, and embeddings are scaled."""
+        layers = []
+        for ent in cfg["layers"]:
+            m, kind = ent["mixer"], ent["type"]
+            if kind == "mingru":
+                mixer, mtype = GruMixerSpec(width=int(m["width"])), "gru"
+                if mixer.width < 1:
+                    raise ValueError("the recurrence needs a width")
+            elif kind in ("attention", "attention_2"):
+                r = m.get("rot") or {}
+                mask = m.get("mask") or {}
+                mixer = PagedMixerSpec(
+                    heads=int(m["heads"]), kv_heads=int(m["kv_heads"]),
+                    qk_dim=int(m["dim"]), v_dim=int(m.get("vdim", m["dim"])),
+                    scale=float(m["scale"]),
+                    rot=RotarySpec(dims=int(r.get("dims", 0) or 0),
+                                   base=float(r.get("base", 10000.0)),
+                                   layout="half"),
+                    out_gate=True, **(
+                        dict(conv=int(m["conv"]), unit_norm=True)
+                        if kind == "attention" else
+                        dict(chunk=int(mask["size"]), unit_sink=True)))
+                if mixer.heads % mixer.kv_heads:
+                    raise ValueError("heads must be a multiple of kv_heads")
+                if mixer.rot.dims % 2 or mixer.rot.dims > mixer.qk_dim:
+                    raise ValueError(
+                        "rotary dims must be even and fit the head")
+                if kind == "attention" and mixer.conv < 1:
+                    raise ValueError("the convolution needs a tap")
+                if kind == "attention_2" and mixer.chunk < 1:
+                    raise ValueError("the chunk size must be positive")
+                mtype = "paged_attention"
+            else:
+                raise NotImplementedError(
+                    f"Fuvuvik mixer type {kind!r} is not implemented")
+            f = ent.get("mlp")
+            if not f:
+                ff = None
+            elif f["kind"] == "dense":
+                ff = FeedForwardSpec(kind="dense", ff=int(f["ff"]),
+                                     act="gelu_tanh", gated=True)
+            else:
+                raise NotImplementedError(
+                    f"Fuvuvik feed-forward kind {f['kind']!r}")
+            layers.append(LayerSpec(mtype, mixer, ff))
+        streams = int(cfg["streams"])
+        if streams < 1:
+            raise ValueError("at least one residual stream")
+        return cls(
+            architecture="Fuvuvik",
+            vocab_size=int(cfg["vocab"]),
+            hidden_size=int(cfg["width"]),
+            num_layers=len(layers),
+            layers=tuple(layers),
+            num_heads=1, num_kv_heads=1, head_dim=8, intermediate_size=0,
+            rms_norm_eps=float(cfg["norm"]["eps"]),
+            max_position_embeddings=int(
+                cfg.get("max_position_embeddings", 1 << 20)),
+            eos_token_id=int(cfg.get("eos_token_id", -1)),
+            fp32_residual=True, streams=streams, token_shift=True,
+            residual_gate=True,
+            embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
+        )
+
+    @classmethod
     def from_hf_config(cls, cfg: dict) -> "ModelSpec":
+        if cfg.get("architecture") == "Fuvuvik" and "architectures" not in cfg:
+            return cls._from_fuvuvik_config(cfg)
         if cfg.get("architecture") == "Makezen" and "architectures" not in cfg:
             return cls._from_makezen_config(cfg)
         if cfg.get("architecture") == "Livasun" and "architectures" not in cfg:

@@ -250,11 +250,13 @@ class KVCache:
         # recurrent mixers: per layer run a matrix state [slots + 1, heads,
         # state, vdim] in fp32 whatever the engine dtype, and the last
         # inputs of the short convolution [slots + 1, taps - 1, channels]
-        # in the engine dtype. One slot per live sequence (max_num_seqs of
-        # them); the extra last slot takes the padded rows of a captured
+        # in the engine dtype; with a token shift also the previous token's
+        # normed row [slots + 1, width] of every run. One slot per live
+        # sequence (max_num_seqs of them); the extra last slot takes the padded rows of a captured
         # decode graph, as pad_block does for the paged pools
         self.ssm_states: list = [None] * self.num_layers
         self.conv_states: list = [None] * self.num_layers
+        self.shift_states: list = [None] * self.num_layers
         self.state_allocator = None
         self.pad_state_slot = -1
         if self.layered and spec.has_state:
@@ -274,13 +276,19 @@ class KVCache:
                 if sh is None:
                     continue
                 heads, n, vdim, crows, cch = sh
-                self.ssm_states[r] = torch.zeros(
-                    (nslots + 1, heads, n, vdim), dtype=torch.float32,
-                    device=device)
+                if heads > 0:
+                    self.ssm_states[r] = torch.zeros(
+                        (nslots + 1, heads, n, vdim), dtype=torch.float32,
+                        device=device)
                 if cch > 0:
                     self.conv_states[r] = torch.zeros(
                         (nslots + 1, crows, cch), dtype=act_dtype,
                         device=device)
+            if spec.token_shift:
+                self.shift_states = [
+                    torch.zeros((nslots + 1, spec.hidden_size),
+                                dtype=act_dtype, device=device)
+                    for _ in range(self.num_layers)]
         # last block reserved as the graph-padding scratch block (see
         # engine/graph_runner.py): padded rows write/read there, never live KV
         self.pad_block = num_blocks - 1

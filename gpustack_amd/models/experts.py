@@ -29,14 +29,24 @@ from ..engine.config import FeedForwardSpec
 
 
 class DenseFF(nn.Module):
-    def __init__(self, width: int, f: FeedForwardSpec, dtype, comm=None):
+    """`extra` further rows of the up projection are handed back beside the
+    block's output (a projection of the same input that someone else
+    needs, a residual gate for instance)."""
+
+    def __init__(self, width: int, f: FeedForwardSpec, dtype, comm=None,
+                 extra: int = 0):
         super().__init__()
         if comm is not None and comm.tp_size > 1:
             raise NotImplementedError("ungated FF is not TP-sharded yet")
         self.act, self.gated, self.ff = f.act, f.gated, f.ff
         # gated: rows [0, ff) are the gate, [ff, 2 ff) the up projection
+        # and the extra rows behind them
+        self.cols = f.ff * (2 if f.gated else 1)
+        self.extra = extra
+        if extra and not f.gated:
+            raise NotImplementedError("extra rows come with the gated form")
         self.up_w = nn.Parameter(
-            torch.empty(f.ff * (2 if f.gated else 1), width, dtype=dtype),
+            torch.empty(self.cols + extra, width, dtype=dtype),
             requires_grad=False)
         self.down_w = nn.Parameter(torch.empty(width, f.ff, dtype=dtype),
                                    requires_grad=False)
@@ -46,7 +56,9 @@ class DenseFF(nn.Module):
         if self.gated:
             g = torch.empty(h.shape[0], self.ff, dtype=h.dtype,
                             device=h.device)
-            ops.act_and_mul(g, u, self.act)
+            ops.act_and_mul(g, u[:, :self.cols], self.act)
+            if self.extra:
+                return F.linear(g, self.down_w), u[:, self.cols:]
             u = g
         else:
             ops.act_inplace(u, self.act)

@@ -77,6 +77,27 @@ class RaggedMeta:
             self._tiles[key] = g
         return g
 
+    @property
+    def single(self) -> bool:
+        """Every sequence brings one row (a decode step)."""
+        return max(self.seq_news, default=1) <= 1
+
+    def scan_chunks(self, size: int):
+        """The batch's rows cut into runs of at most `size` rows of one
+        sequence (ops.build_scan_chunks), or None when no sequence brings
+        more than that."""
+        if max(self.seq_news, default=1) <= size:
+            return None
+        if self._tiles is None:
+            self._tiles = {}
+        key = ("chunks", size)
+        c = self._tiles.get(key)
+        if c is None:
+            c = ops.build_scan_chunks(self.seq_starts, self.seq_news, size,
+                                      self.block_tables.device)
+            self._tiles[key] = c
+        return c
+
     def attn_tiles(self, heads: int, kv_heads: int, maps: int):
         """Workgroup tile list for ops.paged_attention, cached per head
         layout (layers of one model may differ in it)."""

@@ -28,6 +28,11 @@ states. Nothing is kept per token.
   sigmoid(b); each head's output is RMS-normed, weighted and multiplied by
   silu(gate).
 
+* MinGruMixer keeps one value per channel instead of a matrix
+  (ops.gru_scan), S_t = (1 - z_t) S_(t-1) + z_t c_t: one projection gives z
+  | u | gate; z = sigmoid(z + b_z), c = u + b_u + 1/2 where that sum u + b_u
+  is >= 0, else its sigmoid; the output is S_t * silu(gate).
+
 Decays, step sizes, the recurrence and both norms are fp32; the
 projections (library GEMMs) and the convolution run in the engine dtype.
 """
@@ -38,7 +43,7 @@ import torch.nn.functional as F
 from torch import nn
 
 from .. import ops
-from ..engine.config import ScanMixerSpec
+from ..engine.config import GruMixerSpec, ScanMixerSpec
 
 
 def _mk(*shape, dt):
@@ -172,6 +177,33 @@ class GatedDeltaMixer(nn.Module):
         ops.gated_group_norm(g, y, u[:, self.col_gate:self.col_a],
                              self.norm_rows, m.heads, self.eps, 2)
         out = F.linear(g, self.o_w)
+        return self.comm.all_reduce(out) if self.comm is not None else out
+
+
+class MinGruMixer(nn.Module):
+    def __init__(self, width: int, m: GruMixerSpec, dtype, comm=None):
+        super().__init__()
+        if comm is not None and comm.tp_size > 1:
+            raise NotImplementedError(
+                "recurrent mixers are not sharded for tensor parallelism yet")
+        self.m, self.comm = m, comm
+        f32 = torch.float32
+        # rows: z | u | gate
+        self.in_w = _mk(3 * m.width, width, dt=dtype)
+        self.z_b = _mk(m.width, dt=f32)
+        self.u_b = _mk(m.width, dt=f32)
+        self.o_w = _mk(width, m.width, dt=dtype)
+
+    def forward(self, h, meta, state):
+        n = self.m.width
+        rg = meta.ragged
+        u = F.linear(h, self.in_w)
+        y = torch.empty(h.shape[0], n, dtype=h.dtype, device=h.device)
+        ops.gru_scan(y, u, 0, n, 2 * n, self.z_b, self.u_b, state,
+                     rg.seq_first, rg.seq_rows, rg.state_slots, rg.pos32,
+                     chunks=rg.scan_chunks(ops.SCAN_CHUNK) if h.is_cuda
+                     else None)
+        out = F.linear(y, self.o_w)
         return self.comm.all_reduce(out) if self.comm is not None else out
 
 

@@ -68,6 +68,9 @@ def _layered_tensor_plan(model):
         plan.append(("head", model.lm_head, same))
     for i, layer in enumerate(model.layers):
         p = f"l{i}."
+        if hasattr(layer, "port1"):
+            plan += _stream_layer_plan(p, layer)
+            continue
         if hasattr(layer, "mixer") and hasattr(layer, "pre1"):
             plan += _sandwich_ln_layer_plan(p, layer)
             continue
@@ -248,6 +251,49 @@ def _sandwich_ln_layer_plan(p: str, layer):
     return plan
 
 
+def _stream_layer_plan(p: str, layer):
+    """Plan entries of one layer on parallel residual streams with gated
+    sublayers and shifted mixer inputs (models/fuvuvik.py): q, k, v and the
+    head gates (or the recurrence's z, u and gate) fuse into one
+    projection, the feed-forward's gate, up and residual gate into
+    another; stream weights, shifts, biases and convolutions stay fp32."""
+    same = lambda t: t
+    a = layer.mixer
+    plan = []
+    for q, port in (("1", layer.port1), ("2", layer.port2)):
+        if port is not None:
+            plan += [(p + "norm" + q, port.norm, same),
+                     (p + f"hc{q}.in", port.read, same),
+                     (p + f"hc{q}.out", port.write, same),
+                     (p + f"hc{q}.mix", port.mix, same),
+                     (p + f"rg{q}.b", port.gate_b, same)]
+    plan += [(p + "shift", layer.shift, same),
+             (p + "rg1", layer.gate1_w, same), (p + "mix.o", a.o_w, same)]
+    if layer.kind == "gru":
+        n = a.m.width
+        plan += [(p + "mix.z", a.in_w[:n], same),
+                 (p + "mix.x", a.in_w[n:2 * n], same),
+                 (p + "mix.g", a.in_w[2 * n:], same),
+                 (p + "mix.z.b", a.z_b, same), (p + "mix.x.b", a.u_b, same)]
+    else:
+        nq, nk, c = a.nq, a.nk, a.col_gate
+        plan += [(p + "mix.q", a.qkv_w[:nq], same),
+                 (p + "mix.k", a.qkv_w[nq:nq + nk], same),
+                 (p + "mix.v", a.qkv_w[nq + nk:c], same),
+                 (p + "mix.g", a.qkv_w[c:c + a.m.heads], same)]
+        if a.conv_w is not None:
+            plan += [(p + "mix.q.conv", a.conv_w[:nq], same),
+                     (p + "mix.k.conv", a.conv_w[nq:nq + nk], same),
+                     (p + "mix.v.conv", a.conv_w[nq + nk:], same)]
+    m = layer.mlp
+    if m is not None:
+        plan += [(p + "mlp.gate", m.up_w[:m.ff], same),
+                 (p + "mlp.up", m.up_w[m.ff:m.cols], same),
+                 (p + "rg2", m.up_w[m.cols:], same),
+                 (p + "mlp.down", m.down_w, same)]
+    return plan
+
+
 def _routed_ff_plan(p: str, m):
     """Plan entries of a routed expert bank (models/experts.py)."""
     same = lambda t: t
@@ -322,15 +368,26 @@ def _random_init_layered(model, cfg: EngineConfig) -> None:
     1/fan_in), norm and layer-scale weights near 1 / near 0.5, so deep
     random stacks keep O(1) activations."""
     for name, dst, fn in _layered_tensor_plan(model):
+        if ".hc" in name:
+            # stream weights: read and write about evenly, streams mostly
+            # kept apart, so that their sizes stay O(1)
+            t = _gen(tuple(dst.shape), name, cfg.seed, torch.float32,
+                     model.device, std=0.1)
+            if dst.dim() == 2:
+                t = 0.9 * torch.eye(dst.shape[0], device=t.device) + 0.3 * t
+            else:
+                t = t + (1.0 / dst.shape[0] if name.endswith("in") else 0.5)
+            dst.copy_(t.to(dst.dtype))
+            continue
         if dst.dim() == 1 and not name.endswith(("router", "sg")):
             leaf = name.rsplit(".", 1)[-1]
             if leaf in ("b", "sink", "lq1", "lk1", "lq2", "lk2"):
                 base, std = 0.0, 0.3     # biases, sinks, lambda vectors
-            elif leaf in ("vmix", "correction", "dt_bias", "A_log"):
+            elif leaf in ("vmix", "correction", "dt_bias", "A_log", "shift"):
                 # blend weight in (0, 1); small choice corrections; step
                 # sizes around softplus(-1); decay rates around 1
                 base, std = {"vmix": (0.3, 0.05), "correction": (0.0, 0.1),
-                             "dt_bias": (-1.0, 0.5),
+                             "dt_bias": (-1.0, 0.5), "shift": (0.3, 0.2),
                              "A_log": (0.0, 0.5)}[leaf]
             else:
                 base, std = (0.5 if leaf in ("ls1", "ls2") else 1.0), 0.05

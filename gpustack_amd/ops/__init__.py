@@ -688,7 +688,8 @@ def paged_attention(out, q, k_cache, v_cache, block_tables, row_seq, positions,
                     scale: float, maps: int = 1, window: int = 0,
                     keep_first: int = 0, sinks=None, tiles=None,
                     exact: bool = False, max_ctx: int = 0,
-                    slopes=None, softcap: float = 0.0) -> None:
+                    slopes=None, softcap: float = 0.0, chunk: int = 0,
+                    gate=None) -> None:
     """q: [T, A, D], out: [T, A, VW] (A = heads * maps score maps; views
     whose last axis is contiguous). On the
     GPU the MFMA kernel runs for bf16 pools of fitting sizes, the fp32
@@ -696,7 +697,9 @@ def paged_attention(out, q, k_cache, v_cache, block_tables, row_seq, positions,
     `max_ctx` (longest context in the batch, a host number) lets a batch of
     few tiles over long contexts split each tile's keys over workgroups.
     `slopes` (fp32, per head): slope * distance is taken off every scaled
-    score. `softcap` > 0: scaled scores pass softcap * tanh(s / softcap)."""
+    score. `softcap` > 0: scaled scores pass softcap * tanh(s / softcap).
+    `chunk` > 0: keys of the row's own chunk of positions only. `gate`
+    ([T, heads] view in q's dtype): a head's output times sigmoid(gate)."""
     k = _paged_backend(q)
     if k is not None:
         if tiles is None:
@@ -705,6 +708,8 @@ def paged_attention(out, q, k_cache, v_cache, block_tables, row_seq, positions,
         nsplit = 1
         nt = tiles.shape[0]
         span = min(max_ctx, window + keep_first) if window > 0 else max_ctx
+        if chunk > 0:
+            span = min(span, chunk)
         if span >= 512 and 0 < nt < 2048:
             # 1024 workgroups, or up to 2048 while the split stays <= 4 (a
             # wider split pays more for the merge than it gains in
@@ -713,11 +718,12 @@ def paged_attention(out, q, k_cache, v_cache, block_tables, row_seq, positions,
                                 max(1024 // nt, min(4, 2048 // nt))))
         k.paged_attention(out, q, k_cache, v_cache, block_tables, tiles,
                           positions, scale, maps, window, keep_first, sinks,
-                          exact, nsplit, slopes, softcap)
+                          exact, nsplit, slopes, softcap, chunk, gate)
     else:
         torch_ref.paged_attention(out, q, k_cache, v_cache, block_tables,
                                   row_seq, positions, scale, maps, window,
-                                  keep_first, sinks, slopes, softcap)
+                                  keep_first, sinks, slopes, softcap, chunk,
+                                  gate)
 
 
 def head_rope_store(q_out, src, col_q: int, q_heads: int, q_dim: int, q_w,
@@ -839,15 +845,28 @@ def head_norm_store(q_out, qkv, nq: int, nk: int, q_w, k_w, head_dim: int,
                                   k_cache, v_cache, slots, eps)
 
 
+def short_conv(out, src, col0: int, w, b, conv_state, seq_first, seq_rows,
+               state_slots, row_seq, pos32, silu: bool = True,
+               single: bool = False) -> None:
+    """Short causal convolution per channel, with or without SiLU
+    (torch_ref.short_conv has the semantics). `single` (a host-side hint):
+    every sequence brings one row; the slot moves on in the same launch."""
+    if src.is_cuda:
+        # the kernel ships in both libraries: whichever is loaded
+        k = _STATE or _STREAMS or _load_streams()
+        k.short_conv(out, src, col0, w, b, conv_state, seq_first, seq_rows,
+                     state_slots, row_seq, pos32, silu, single)
+    else:
+        torch_ref.short_conv(out, src, col0, w, b, conv_state, seq_first,
+                             seq_rows, state_slots, pos32, silu)
+
+
 def causal_conv_silu(out, src, col0: int, w, b, conv_state, seq_first,
                      seq_rows, state_slots, row_seq, pos32) -> None:
-    k = _state_backend(src)
-    if k is not None:
-        k.causal_conv_silu(out, src, col0, w, b, conv_state, seq_first,
-                           seq_rows, state_slots, row_seq, pos32)
-    else:
-        torch_ref.causal_conv_silu(out, src, col0, w, b, conv_state,
-                                   seq_first, seq_rows, state_slots, pos32)
+    if src.is_cuda:
+        _load_state()       # models that call this run on that library
+    short_conv(out, src, col0, w, b, conv_state, seq_first, seq_rows,
+               state_slots, row_seq, pos32)
 
 
 def state_scan(y, src, col_x: int, col_b: int, col_c: int, dt_src,
@@ -908,3 +927,112 @@ def delta_scan(y, src, col_q: int, col_k: int, col_v: int, gate_src,
                              col_b, heads, groups, n_state, vdim, dt_bias,
                              a_log, state, seq_first, seq_rows, state_slots,
                              pos32)
+
+
+# --- parallel residual streams, token shift, gated recurrence --------------
+# ops/csrc/hyperrows32.hip, gru_scan.hip and short_conv.hip in
+# `_hip_streams.so`.
+
+_STREAMS = None
+
+
+def _load_streams():
+    """Load `_hip_streams.so` (stream rows, token shift, gated recurrence,
+    short convolution), compiling it in-tree first when no built library is
+    there."""
+    global _STREAMS
+    if _STREAMS is not None:
+        return _STREAMS
+    import importlib.util
+
+    from .build import STREAMS_SO_PATH, build_streams
+
+    if not STREAMS_SO_PATH.exists():
+        build_streams()
+    spec = importlib.util.spec_from_file_location(
+        "gpustack_amd.ops._hip_streams", STREAMS_SO_PATH)
+    mod = importlib.util.module_from_spec(spec)
+    spec.loader.exec_module(mod)
+    _STREAMS = mod
+    return mod
+
+
+def _streams_backend(t: torch.Tensor):
+    return _load_streams() if t.is_cuda else None
+
+
+def embed_streams(x, tokens, embed, scale: float) -> None:
+    k = _streams_backend(x)
+    if k is not None:
+        k.embed_streams(x, tokens, embed, scale)
+    else:
+        torch_ref.embed_streams(x, tokens, embed, scale)
+
+
+def stream_step(x, a, gate, gate_b, mix, out_w, in_w, norm_w, eps: float, h,
+                shift=None) -> None:
+    """Close one sublayer on the streams and open the next
+    (torch_ref.stream_step has the semantics). `shift` = (hs, mu, state,
+    row_seq, state_slots, pos32), for batches of single rows: the token
+    shift of h runs in the same launch."""
+    k = _streams_backend(x)
+    if k is not None:
+        k.stream_step(x, a, gate, gate_b, mix, out_w, in_w, norm_w, eps, h,
+                      *(shift or (None,) * 6))
+        return
+    torch_ref.stream_step(x, a, gate, gate_b, mix, out_w, in_w, norm_w, eps, h)
+    if shift is not None:
+        hs, mu, state, row_seq, slots, pos32 = shift
+        one = torch.ones_like(row_seq)
+        torch_ref.token_shift(hs, h, mu, state,
+                              torch.arange(h.shape[0], device=h.device), one,
+                              slots[row_seq.long()], pos32)
+
+
+def token_shift(hs, h, mu, state, seq_first, seq_rows, state_slots, row_seq,
+                pos32) -> None:
+    k = _streams_backend(h)
+    if k is not None:
+        k.token_shift(hs, h, mu, state, seq_first, seq_rows, state_slots,
+                      row_seq, pos32)
+    else:
+        torch_ref.token_shift(hs, h, mu, state, seq_first, seq_rows,
+                              state_slots, pos32)
+
+
+SCAN_CHUNK = 64   # rows of one sequence a workgroup of the scan walks
+
+
+def build_scan_chunks(seq_starts, seq_news, size: int, device):
+    """Runs of at most `size` rows of one sequence in order, for scans that
+    split a prompt over workgroups: int32 [n, 4] = first row, rows,
+    sequence, list index of the sequence's first run."""
+    import numpy as np
+
+    parts, n = [], 0
+    for i, (st, new) in enumerate(zip(seq_starts, seq_news)):
+        lo = np.arange(0, new, size)
+        t = np.empty((lo.size, 4), dtype=np.int32)
+        t[:, 0] = st + lo
+        t[:, 1] = np.minimum(size, new - lo)
+        t[:, 2] = i
+        t[:, 3] = n
+        n += lo.size
+        parts.append(t)
+    c = np.concatenate(parts) if parts else np.empty((0, 4), dtype=np.int32)
+    return torch.from_numpy(c).to(device)
+
+
+def gru_scan(y, src, col_z: int, col_u: int, col_g: int, z_b, u_b, state,
+             seq_first, seq_rows, state_slots, pos32, chunks=None) -> None:
+    """Gated recurrence with one state value per channel
+    (torch_ref.gru_scan has the semantics). `chunks` (build_scan_chunks; a
+    prompt): rows are split over workgroups, whose partial recurrences are
+    joined; None: one workgroup walks all rows of a sequence."""
+    k = _streams_backend(src)
+    if k is not None:
+        k.gru_scan(y, src, col_z, col_u, col_g, z_b, u_b, state, seq_first,
+                   seq_rows, state_slots, pos32, chunks)
+    else:
+        torch_ref.gru_scan(y, src, col_z, col_u, col_g, z_b, u_b, state,
+                           seq_first, seq_rows, state_slots, pos32)

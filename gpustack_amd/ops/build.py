@@ -34,10 +34,17 @@ PAGED_SOURCES = ["rowmix32.hip", "roperows32.hip", "ragged_attn.hip",
                  "resid32.hip", "paged_bindings.cpp"]
 
 # layer-norm fp32-stream row kernels, head-norm cache write, scored routing
-# and the recurrent mixers (page-wise value stores come with rowmix32.hip)
+# and the recurrent mixers with their short convolution (page-wise value
+# stores come with rowmix32.hip)
 STATE_SO_PATH = PKG_DIR / "_hip_state.so"
 STATE_SOURCES = ["lnrows32.hip", "state_scan.hip", "delta_scan.hip",
-                 "rowmix32.hip", "state_bindings.cpp"]
+                 "short_conv.hip", "rowmix32.hip", "state_bindings.cpp"]
+
+# rows of parallel residual streams, token shift, gated recurrence, short
+# convolution
+STREAMS_SO_PATH = PKG_DIR / "_hip_streams.so"
+STREAMS_SOURCES = ["hyperrows32.hip", "gru_scan.hip", "short_conv.hip",
+                   "stream_bindings.cpp"]
 
 
 def _torch_paths():
@@ -161,6 +168,13 @@ def build_state(verbose: bool = False, force: bool = True) -> Path:
                         verbose, force)
 
 
+def build_streams(verbose: bool = False, force: bool = True) -> Path:
+    """Compile the parallel-stream / gated recurrence family into
+    `_hip_streams.so`."""
+    return _build_small("_hip_streams", STREAMS_SOURCES, STREAMS_SO_PATH,
+                        verbose, force)
+
+
 def _build_small(ext_name: str, sources: list[str], so_path: Path,
                  verbose: bool, force: bool) -> Path:
     """Compile one small extension, its files in parallel. Objects are
@@ -172,7 +186,7 @@ def _build_small(ext_name: str, sources: list[str], so_path: Path,
     build_dir = CSRC / f".build{ext_name}"
     build_dir.mkdir(exist_ok=True)
     newest = max((CSRC / s).stat().st_mtime
-                 for s in sources + ["common.h"])
+                 for s in sources + ["common.h", "short_conv_binding.h"])
     if (so_path.exists() and not force
             and so_path.stat().st_mtime >= newest):
         return so_path
@@ -213,10 +227,14 @@ if __name__ == "__main__":
     elif "--state" in sys.argv:
         build_state(verbose=True)
         print(f"built {STATE_SO_PATH}")
+    elif "--streams" in sys.argv:
+        build_streams(verbose=True)
+        print(f"built {STREAMS_SO_PATH}")
     else:
         build(verbose=True, force="--force" in sys.argv)
         build_latent(verbose=True)
         build_paged(verbose=True)
         build_state(verbose=True)
+        build_streams(verbose=True)
         print(f"built {SO_PATH} {LATENT_SO_PATH} {PAGED_SO_PATH} "
-              f"{STATE_SO_PATH}")
+              f"{STATE_SO_PATH} {STREAMS_SO_PATH}")

@@ -11,9 +11,9 @@ void sandwich_add_norm_launch(float*, const void*, const float*, float, const fl
 void rotary_norm_store_launch(void*, const void*, long, int, int, int, const float*, const float*, const float*, int, const int*, int, void*, void*, const long*, long, int, int, int, int, float, int, int, int, hipStream_t);
 void value_page_store_launch(const void*, long, int, void*, const long*, long, const int*, int, int, int, int, int, int, hipStream_t);
 void diff_combine_launch(void*, const float*, const float*, float, float, long, int, int, hipStream_t);
-void act_and_mul_launch(void*, const void*, long, int, int, int, hipStream_t);
+void act_and_mul_launch(void*, const void*, long, long, int, int, int, hipStream_t);
 void argmax_f32_launch(long*, const float*, int, int, hipStream_t);
-void paged_attention_launch(void*, const void*, const void*, const void*, const int*, const int*, const int*, const float*, const float*, float, float, long, long, long, long, int, int, int, int, int, int, int, int, int, int, int, int, int, int, int, int, int, int, int, float*, float*, hipStream_t);
+void paged_attention_launch(void*, const void*, const void*, const void*, const int*, const int*, const int*, const float*, const float*, float, float, long, long, long, long, int, int, int, int, int, int, int, int, int, int, int, int, int, int, int, int, const void*, long, int, int, int, int, float*, float*, hipStream_t);
 void head_rope_store_launch(void*, const void*, long, int, int, int, const float*, int, int, int, int, int, const float*, int, int, int, const float*, int, int, float, const int*, void*, void*, const long*, long, int, int, float, int, int, int, hipStream_t);
 void dual_rms_mix_launch(void*, const void*, const float*, const void*, const float*, int, int, float, int, hipStream_t);
 void head_gate_launch(void*, const void*, const void*, long, int, int, int, int, int, hipStream_t);
@@ -183,7 +183,8 @@ void paged_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                      Tensor block_tables, Tensor tiles, Tensor pos32,
                      double scale, long maps, long window, long keep_first,
                      OptTensor sinks, bool exact, long nsplit,
-                     OptTensor slopes, double softcap) {
+                     OptTensor slopes, double softcap, long chunk,
+                     OptTensor gate) {
   chk(block_tables, "block_tables", at::kInt);
   chk(tiles, "tiles", at::kInt);
   chk(pos32, "pos32", at::kInt);
@@ -210,7 +211,17 @@ void paged_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
               "head size unsupported");
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(1) >= 1 &&
               tiles.dim() == 2 && tiles.size(1) == 6 && pos32.numel() == T);
-  TORCH_CHECK(window >= 0 && keep_first >= 0);
+  TORCH_CHECK(window >= 0 && keep_first >= 0 && chunk >= 0);
+  const void* gp = nullptr;
+  long g_st = 0;
+  if (gate.has_value()) {
+    TORCH_CHECK(gate->is_cuda() && gate->scalar_type() == q.scalar_type() &&
+                gate->dim() == 2 && gate->size(0) == T && gate->size(1) == H &&
+                (H == 1 || gate->stride(1) == 1) && gate->stride(0) >= 0,
+                "gate must be [T, heads] rows in q's dtype");
+    gp = gate->data_ptr();
+    g_st = gate->stride(0);
+  }
   const float* sp = nullptr;
   if (sinks.has_value()) {
     chk(*sinks, "sinks", at::kFloat);
@@ -243,7 +254,8 @@ void paged_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                          G, BS,
                          (int)maps, H / G, (int)block_tables.size(0),
                          (int)block_tables.size(1), (int)k_cache.size(0),
-                         (int)window, (int)keep_first, q_bf, out_bf,
+                         (int)window, (int)keep_first, (int)chunk, gp, g_st,
+                         q_bf, out_bf,
                          exact ? 1 : 0, (int)nsplit, wa, wm, cur_stream(q));
   HIP_CHECK_LAST();
 }
@@ -269,11 +281,14 @@ void diff_combine(Tensor out, Tensor a, Tensor lam, double diff, double eps) {
 }
 
 void act_and_mul(Tensor out, Tensor gu, long mode) {
-  const int bf = act_kind(gu, "gu");
-  TORCH_CHECK(act_kind(out, "out") == bf && gu.dim() == 2 && out.dim() == 2);
-  TORCH_CHECK(out.size(0) == gu.size(0) && gu.size(1) == 2 * out.size(1));
+  // gu: rows, maybe strided (the first columns of a wider product)
+  const int bf = act_kind(out, "out");
+  TORCH_CHECK(gu.is_cuda() && gu.scalar_type() == out.scalar_type() &&
+              gu.dim() == 2 && out.dim() == 2);
+  TORCH_CHECK(out.size(0) == gu.size(0) && gu.size(1) == 2 * out.size(1) &&
+              gu.stride(1) == 1 && gu.stride(0) >= gu.size(1));
   TORCH_CHECK(mode >= 0 && mode <= 3);
-  act_and_mul_launch(out.data_ptr(), gu.data_ptr(), out.size(0),
+  act_and_mul_launch(out.data_ptr(), gu.data_ptr(), gu.stride(0), out.size(0),
                      (int)out.size(1), (int)mode, bf, cur_stream(gu));
   HIP_CHECK_LAST();
 }
@@ -285,9 +300,10 @@ void chk_rope_side(const char* name, long col, long heads, long dim,
   TORCH_CHECK(heads >= 0 && (heads == 0 || (dim >= 1 && col >= 0 &&
               col + heads * dim <= width)), name, " columns outside the row");
   if (heads == 0) return;
+  TORCH_CHECK(nd >= 0 && nd <= dim, name, " normed channels outside the head");
   if (w.has_value()) {
     chk(*w, name, at::kFloat);
-    TORCH_CHECK(nd >= 1 && nd <= dim && w->numel() == nd, name,
+    TORCH_CHECK(nd >= 1 && w->numel() == nd, name,
                 " norm weight does not fit the normed channels");
   }
   TORCH_CHECK(rot0 < 0 || half == 0 || rot0 + 2 * half <= dim, name,
@@ -439,7 +455,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("tiles"), py::arg("pos32"), py::arg("scale"), py::arg("maps"),
         py::arg("window"), py::arg("keep_first"), py::arg("sinks"),
         py::arg("exact"), py::arg("nsplit"), py::arg("slopes") = py::none(),
-        py::arg("softcap") = 0.0);
+        py::arg("softcap") = 0.0, py::arg("chunk") = 0,
+        py::arg("gate") = py::none());
   m.def("paged_attention_uses_mfma", &paged_attention_uses_mfma);
   m.def("diff_combine", &diff_combine);
   m.def("head_rope_store", &head_rope_store);

@@ -4,14 +4,16 @@
 //
 // over the visible keys j of row t's sequence, read through its block
 // table: j <= pos(t), and with a window also (pos(t) - j < window or
-// j < keep_first). a runs over heads * maps SCORE MAPS (a = head * maps +
+// j < keep_first), or, in chunks, only keys of the row's own chunk of
+// positions, j >= pos(t) - pos(t) mod chunk. a runs over heads * maps SCORE MAPS (a = head * maps +
 // map): map m of a head reads channels [m*D, (m+1)*D) of its kv head's key
 // row, and all maps of a head weight the same value rows — two maps per
 // head are the two halves of differential attention, combined afterwards.
 // A per-head sink logit may join the denominator (no key, no value), and a
 // per-head slope times the distance pos(t) - j may be taken off the scaled
 // score (positions without rotation); a tanh cap may bound the scaled
-// score. q and out are [T, A, *] views with a contiguous last axis.
+// score; a sigmoid gate per row and head may multiply the output. q and out
+// are [T, A, *] views with a contiguous last axis.
 //
 // Pools: keys [nblocks, G, BS, KW] with KW = maps * D (rotated at write
 // time), values with every page transposed, [nblocks, G, VW, BS], so both
@@ -21,9 +23,11 @@
 // A workgroup takes a tile of up to 16 (row, map) pairs that share one key
 // stream — same sequence, same kv head, same map (host-built list: 16 rows
 // x 1 map inside prompts, rows x the query heads of a kv group for decode
-// rows) — and walks that stream once for all of them. Key tiles that lie
-// wholly outside every pair's window (and past the kept first keys) are
-// skipped, so a windowed layer costs its window, not its context.
+// rows) — and walks that stream once for all of them. Each pair sees the
+// keys from a lower bound of its own up to its position, plus the kept first
+// keys; the walk visits the key tiles of the kept keys and those from the
+// pairs' smallest bound on, so a windowed or chunked layer costs its window
+// or chunk, not its context.
 //
 // Two paths. The MFMA path (bf16 q and pools, BS = 16, D % 32 == 0, VW %
 // 16 == 0) runs both products on v_mfma_f32_16x16x32_bf16 with fp32
@@ -67,13 +71,15 @@ struct AttnArgs {
   long q_st, q_sa;           // element strides of q [T, A, D]: row, score map
   long o_st, o_sa;           // and of out [T, A, VW]
   int T, A, D, VW, KW, G, BS, maps, rep;   // rep = heads / kv heads
-  int nseq, maxb, nblocks, window, keep_first;
+  int nseq, maxb, nblocks, window, keep_first, chunk;
+  const void* gate;          // [T, A / maps] view in q's dtype, or null
+  long g_st;
 };
 
 // Decodes and validates a tile; false = skip the tile untouched.
 DEVICE_INLINE bool tile_setup(const AttnArgs& p, int tile, int* e_pos,
-                              int* e_row, int* e_a, int& n_ent, int& seq,
-                              int& g, int& koff) {
+                              int* e_lo, int* e_row, int* e_a, int& n_ent,
+                              int& seq, int& g, int& koff) {
   const int* tl = p.tiles + (long)tile * 6;
   const int row0 = tl[0], nrows = tl[1], a0 = tl[2], n_a = tl[3];
   const int a_step = tl[5];
@@ -87,21 +93,48 @@ DEVICE_INLINE bool tile_setup(const AttnArgs& p, int tile, int* e_pos,
   koff = (a0 % p.maps) * p.D;
   if (g >= p.G) return false;
   if (threadIdx.x < G16) {
-    int ps = -1, row = 0, a = 0;
+    int ps = -1, lo = 1 << 30, row = 0, a = 0;
     if ((int)threadIdx.x < n_ent) {
       row = row0 + threadIdx.x / n_a;
       a = a0 + (threadIdx.x % n_a) * a_step;
       ps = min(max(p.pos32[row], 0), p.maxb * p.BS - 1);
+      lo = p.window > 0 ? max(0, ps - p.window + 1) : 0;
+      if (p.chunk > 0) lo = max(lo, ps - ps % p.chunk);
     }
     e_pos[threadIdx.x] = ps;
+    e_lo[threadIdx.x] = lo;
     e_row[threadIdx.x] = row;
     e_a[threadIdx.x] = a;
   }
   return true;
 }
 
-DEVICE_INLINE bool key_visible(int j, int pos, int window, int keep_first) {
-  return j <= pos && (window <= 0 || pos - j < window || j < keep_first);
+DEVICE_INLINE bool key_visible(int j, int pos, int lo, int keep_first) {
+  return j <= pos && (j >= lo || j < keep_first);
+}
+
+// The key tiles of KT keys a tile of pairs visits: those of the kept first
+// keys, [0, kept), then [from, end). Position v of the walk is tile
+// v < kept ? v : v - kept + from, v in [0, n).
+struct KeyWalk {
+  int kept, from, n;
+  DEVICE_INLINE int tile(int v) const { return v < kept ? v : v - kept + from; }
+};
+
+DEVICE_INLINE KeyWalk key_walk(int lo, int jmax, int keep_first, int KT) {
+  KeyWalk w;
+  const int end = jmax / KT + 1;
+  w.from = lo / KT;
+  w.kept = min((keep_first + KT - 1) / KT, w.from);
+  w.n = w.kept + end - w.from;
+  return w;
+}
+
+template <typename TG>
+DEVICE_INLINE float head_gate_of(const AttnArgs& p, int row, int a) {
+  if (p.gate == nullptr) return 1.f;
+  const float z = ldf((const TG*)p.gate + (long)row * p.g_st + a / p.maps);
+  return 1.0f / (1.0f + expf(-z));
 }
 
 DEVICE_INLINE float scaled_score(float dot, const AttnArgs& p) {
@@ -124,27 +157,26 @@ __global__ __launch_bounds__(THREADS) void paged_attn_exact_kernel(
   float* ps = vs + KT * VS;           // [16][KT]
   float* als = ps + G16 * KT;         // [16]
   float* lsum = als + G16;            // [16]
-  __shared__ int e_pos[G16], e_row[G16], e_a[G16];
+  __shared__ int e_pos[G16], e_lo[G16], e_row[G16], e_a[G16];
 
   int n_ent, seq, g, koff;
-  if (!tile_setup(p, blockIdx.x, e_pos, e_row, e_a, n_ent, seq, g, koff))
+  if (!tile_setup(p, blockIdx.x, e_pos, e_lo, e_row, e_a, n_ent, seq, g, koff))
     return;
   __syncthreads();
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  int jmax = -1, jmin = 1 << 30;
+  int jmax = -1, lo = 1 << 30;
 #pragma unroll
   for (int e = 0; e < G16; ++e) {
     jmax = max(jmax, e_pos[e]);
-    if (e_pos[e] >= 0) jmin = min(jmin, e_pos[e]);
+    lo = min(lo, e_lo[e]);
   }
-  const int lo = p.window > 0 ? max(0, jmin - p.window + 1) : 0;
   for (int e = wave; e < G16; e += 4) {
     const bool ok = e < n_ent;
     const TQ* qp = q + (long)e_row[e] * p.q_st + (long)e_a[e] * p.q_sa;
     for (int r = lane; r < D; r += 64) qs[e * D + r] = ok ? ldf(qp + r) : 0.f;
   }
   const int e_s = tid >> 4, kk = tid & 15;
-  const int my_pos = e_pos[e_s];
+  const int my_pos = e_pos[e_s], my_lo = e_lo[e_s];
   float m_run = -INFINITY, l_run = 0.f;
   if (p.sinks != nullptr && my_pos >= 0) {
     m_run = p.sinks[e_a[e_s] / p.maps];
@@ -159,8 +191,9 @@ __global__ __launch_bounds__(THREADS) void paged_attn_exact_kernel(
 
   const int* bt = p.block_tables + (long)seq * p.maxb;
   const int BS = p.BS;
-  for (int k0 = 0; k0 <= jmax; k0 += KT) {
-    if (p.window > 0 && k0 >= p.keep_first && k0 + KT - 1 < lo) continue;
+  const KeyWalk walk = key_walk(lo, jmax, p.keep_first, KT);
+  for (int v = 0; v < walk.n; ++v) {
+    const int k0 = walk.tile(v) * KT;
     __syncthreads();   // previous tile fully consumed (and qs written)
     for (int k = wave; k < KT; k += 4) {
       const int j = k0 + k;
@@ -200,7 +233,7 @@ __global__ __launch_bounds__(THREADS) void paged_attn_exact_kernel(
 #pragma unroll
     for (int u = 0; u < KT / 16; ++u) {
       const int j = k0 + kk + 16 * u;
-      s[u] = key_visible(j, my_pos, p.window, p.keep_first)
+      s[u] = key_visible(j, my_pos, my_lo, p.keep_first)
                  ? scaled_score(s[u], p) - slope * (float)(my_pos - j)
                  : -INFINITY;
       mx = fmaxf(mx, s[u]);
@@ -254,7 +287,8 @@ __global__ __launch_bounds__(THREADS) void paged_attn_exact_kernel(
     const int e = wave + 4 * i;
     if (e >= n_ent) continue;
     const float l = lsum[e];
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    const float inv = (l > 0.f ? 1.0f / l : 0.f) *
+                      head_gate_of<TQ>(p, e_row[e], e_a[e]);
     TO* op = out + (long)e_row[e] * p.o_st + (long)e_a[e] * p.o_sa;
 #pragma unroll
     for (int j = 0; j < NJ; ++j) {
@@ -293,21 +327,20 @@ __global__ __launch_bounds__(THREADS) void paged_attn_mfma_kernel(
   float* Ss = reinterpret_cast<float*>(Pl + G16 * MPS);  // [16][MSS]
   float* als = Ss + G16 * MSS;                        // [16]
   float* lsum = als + G16;                            // [16]
-  __shared__ int e_pos[G16], e_row[G16], e_a[G16];
+  __shared__ int e_pos[G16], e_lo[G16], e_row[G16], e_a[G16];
 
   int n_ent, seq, g, koff;
-  if (!tile_setup(p, blockIdx.x, e_pos, e_row, e_a, n_ent, seq, g, koff))
+  if (!tile_setup(p, blockIdx.x, e_pos, e_lo, e_row, e_a, n_ent, seq, g, koff))
     return;
   __syncthreads();
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int lc = lane & 15, lg = lane >> 4;
-  int jmax = -1, jmin = 1 << 30;
+  int jmax = -1, lo = 1 << 30;
 #pragma unroll
   for (int e = 0; e < G16; ++e) {
     jmax = max(jmax, e_pos[e]);
-    if (e_pos[e] >= 0) jmin = min(jmin, e_pos[e]);
+    lo = min(lo, e_lo[e]);
   }
-  const int lo = p.window > 0 ? max(0, jmin - p.window + 1) : 0;
   for (int e = wave; e < G16; e += 4) {
     const bool ok = e < n_ent;
     const unsigned short* qp =
@@ -317,7 +350,7 @@ __global__ __launch_bounds__(THREADS) void paged_attn_mfma_kernel(
   }
 
   const int e_s = tid >> 4, kk = tid & 15;    // softmax role
-  const int my_pos = e_pos[e_s];
+  const int my_pos = e_pos[e_s], my_lo = e_lo[e_s];
   const int nsplit = gridDim.y, split = blockIdx.y;
   float m_run = -INFINITY, l_run = 0.f;
   if (p.sinks != nullptr && my_pos >= 0 && split == 0) {
@@ -331,12 +364,11 @@ __global__ __launch_bounds__(THREADS) void paged_attn_mfma_kernel(
 
   const int* bt = p.block_tables + (long)seq * p.maxb;
   const int last_page = jmax >> 4;
-  const int ntk = jmax / MKT + 1;                       // key tiles
-  const int per = (ntk + nsplit - 1) / nsplit;
-  const int t_end = min(ntk, (split + 1) * per);
-  for (int kt = split * per; kt < t_end; ++kt) {
-    const int k0 = kt * MKT;
-    if (p.window > 0 && k0 >= p.keep_first && k0 + MKT - 1 < lo) continue;
+  const KeyWalk walk = key_walk(lo, jmax, p.keep_first, MKT);
+  const int per = (walk.n + nsplit - 1) / nsplit;
+  const int v_end = min(walk.n, (split + 1) * per);
+  for (int v = split * per; v < v_end; ++v) {
+    const int k0 = walk.tile(v) * MKT;
     __syncthreads();   // Ql staged / previous tile's Pl and als consumed
     {
       // scores: this wave's 16 keys; keys past jmax re-read key jmax (their
@@ -364,7 +396,7 @@ __global__ __launch_bounds__(THREADS) void paged_attn_mfma_kernel(
 #pragma unroll
       for (int u = 0; u < 4; ++u) {
         const int j = k0 + kk + 16 * u;
-        sv[u] = key_visible(j, my_pos, p.window, p.keep_first)
+        sv[u] = key_visible(j, my_pos, my_lo, p.keep_first)
                     ? scaled_score(Ss[e_s * MSS + kk + 16 * u], p) -
                           slope * (float)(my_pos - j)
                     : -INFINITY;
@@ -447,7 +479,8 @@ __global__ __launch_bounds__(THREADS) void paged_attn_mfma_kernel(
     const int e = lg * 4 + r;
     if (e >= n_ent) continue;
     const float l = lsum[e];
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    const float inv = (l > 0.f ? 1.0f / l : 0.f) *
+                      head_gate_of<unsigned short>(p, e_row[e], e_a[e]);
     TO* op = out + (long)e_row[e] * p.o_st + (long)e_a[e] * p.o_sa;
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
@@ -485,8 +518,9 @@ __global__ __launch_bounds__(MERGE_THREADS) void paged_attn_merge_kernel(
     const float* ml = ws_ml + ((base + s) * G16 + e) * 2;
     if (ml[0] != -INFINITY) L += ml[1] * __expf(ml[0] - M);
   }
-  const float inv = L > 0.f ? 1.0f / L : 0.f;
   const int row = row0 + e / n_a, a = a0 + (e % n_a) * a_step;
+  const float inv = (L > 0.f ? 1.0f / L : 0.f) *
+                    head_gate_of<unsigned short>(p, row, a);
   TO* op = out + (long)row * p.o_st + (long)a * p.o_sa;
   for (int ch = threadIdx.x; ch < VW; ch += MERGE_THREADS) {
     float v = 0.f;
@@ -580,7 +614,8 @@ void paged_attention_launch(void* out, const void* q, const void* k_cache,
                             long o_st, long o_sa, int ntiles, int T,
                             int A, int D, int VW, int KW, int G, int BS,
                             int maps, int rep, int nseq, int maxb, int nblocks,
-                            int window, int keep_first, int q_bf, int out_bf,
+                            int window, int keep_first, int chunk,
+                            const void* gate, long g_st, int q_bf, int out_bf,
                             int force_exact, int nsplit, float* ws_acc,
                             float* ws_ml, hipStream_t s) {
   if (ntiles == 0) return;
@@ -591,7 +626,7 @@ void paged_attention_launch(void* out, const void* q, const void* k_cache,
   p.sinks = sinks; p.slopes = slopes; p.scale = scale; p.T = T; p.A = A; p.D = D; p.VW = VW;
   p.KW = KW; p.G = G; p.BS = BS; p.maps = maps; p.rep = rep; p.nseq = nseq;
   p.maxb = maxb; p.nblocks = nblocks; p.window = window;
-  p.keep_first = keep_first;
+  p.keep_first = keep_first; p.chunk = chunk; p.gate = gate; p.g_st = g_st;
   if (!force_exact && paged_attn_uses_mfma(q_bf, BS, D, VW)) {
     if (out_bf)
       dispatch_mfma<unsigned short>(out, q, k_cache, v_cache, p, ntiles, nsplit, ws_acc, ws_ml, s);

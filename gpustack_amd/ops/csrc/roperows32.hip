@@ -2,8 +2,8 @@
 // one by one (gfx950).
 //
 //   head_rope_store : per head of a q side and a k side of one projection
-//                     row: RMS norm of the head's first channels with a
-//                     weight vector shared by the heads, then rotation of a
+//                     row: RMS norm of the head's first channels with or
+//                     without a weight vector shared by the heads, then rotation of a
 //                     channel range (pairs (i, i + half) or (2i, 2i + 1),
 //                     cos / sin times an amplitude); q heads out, k heads
 //                     into their page rows, values into the transposed
@@ -37,8 +37,8 @@ struct RopeArgs {
   int col_q, q_heads, q_dim, q_nd, q_rot0;
   int col_k, k_heads, k_dim, k_nd, k_rot0;
   int col_v;                 // < 0: values are the key heads' first VW channels
-  const float* q_w;          // [q_nd] or null
-  const float* k_w;          // [k_nd] or null
+  const float* q_w;          // [q_nd], or null: unit heads (q_nd 0: no norm)
+  const float* k_w;          // [k_nd] likewise
   const float* inv_freq;     // [half]
   int half, half_layout;
   float amp, eps;
@@ -77,7 +77,7 @@ __global__ __launch_bounds__(ROW_THREADS) void head_rope_store_kernel(
   const TS* row = src + (long)t * p.ld_src + (is_k ? p.col_k : p.col_q) +
                   (long)hd * dim;
   float inv = 1.f;
-  if (w != nullptr) {
+  if (nd > 0) {
     float ss = 0.f;
     for (int c = lane; c < nd; c += 64) {
       const float v = ld(row + c);
@@ -99,7 +99,7 @@ __global__ __launch_bounds__(ROW_THREADS) void head_rope_store_kernel(
   const int G = p.k_heads;
   for (int c = lane; c < dim; c += 64) {
     float v = ld(row + c);
-    if (w != nullptr && c < nd) v = v * inv * w[c];
+    if (c < nd) v = w != nullptr ? v * inv * w[c] : v * inv;
     const int r = c - rot0;
     if (rot0 >= 0 && r >= 0 && r < 2 * half) {
       int i, pc;
@@ -114,7 +114,7 @@ __global__ __launch_bounds__(ROW_THREADS) void head_rope_store_kernel(
         pc = lower ? c + 1 : c - 1;
       }
       float o = ld(row + pc);
-      if (w != nullptr && pc < nd) o = o * inv * w[pc];
+      if (pc < nd) o = w != nullptr ? o * inv * w[pc] : o * inv;
       const float cs = cs_tab[i], sn = cs_tab[half + i];
       v = lower ? v * cs - o * sn : v * cs + o * sn;
     }
@@ -173,15 +173,14 @@ __global__ __launch_bounds__(ROW_THREADS) void head_rope_store_vec_kernel(
   {
     // every lane walks the shuffles; heads without a norm add nothing
     float ss = 0.f;
-    if (w != nullptr)
-      for (int c = sub * 8; c < min(nd, dim); c += LPH * 8) {
-        const u16x8 v = *reinterpret_cast<const u16x8*>(row + c);
+    for (int c = sub * 8; c < min(nd, dim); c += LPH * 8) {
+      const u16x8 v = *reinterpret_cast<const u16x8*>(row + c);
 #pragma unroll
-        for (int k = 0; k < 8; ++k) { const float f = bf2f(v[k]); ss += f * f; }
-      }
+      for (int k = 0; k < 8; ++k) { const float f = bf2f(v[k]); ss += f * f; }
+    }
 #pragma unroll
     for (int m = LPH / 2; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, WAVE_SIZE);
-    if (w != nullptr) inv = 1.0f / sqrtf(ss / (float)nd + p.eps);
+    if (nd > 0) inv = 1.0f / sqrtf(ss / (float)nd + p.eps);
   }
   if (!active) return;
   long blk = 0;
@@ -197,7 +196,10 @@ __global__ __launch_bounds__(ROW_THREADS) void head_rope_store_vec_kernel(
     const u16x8 v = *reinterpret_cast<const u16x8*>(row + c);
 #pragma unroll
     for (int k = 0; k < 8; ++k) f[k] = bf2f(v[k]);
-    if (w != nullptr && c < nd) {
+    if (c < nd && w == nullptr) {
+#pragma unroll
+      for (int k = 0; k < 8; ++k) f[k] *= inv;
+    } else if (c < nd) {
       const f32x4 w0 = *reinterpret_cast<const f32x4*>(w + c);
       const f32x4 w1 = *reinterpret_cast<const f32x4*>(w + c + 4);
 #pragma unroll
@@ -437,10 +439,10 @@ void head_rope_store_launch(void* q_out, const void* src, long ld_src,
   const size_t tab = (size_t)2 * half * sizeof(float);
   auto m8 = [](long v) { return v % 8 == 0; };
   const bool q_ok = q_heads == 0 ||
-      (m8(col_q) && m8(q_dim) && (q_w == nullptr || m8(q_nd)) &&
+      (m8(col_q) && m8(q_dim) && m8(q_nd) &&
        (q_rot0 < 0 || m8(q_rot0)) && (uintptr_t)q_out % 16 == 0);
   const bool k_ok = k_heads == 0 ||
-      (m8(col_k) && m8(k_dim) && (k_w == nullptr || m8(k_nd)) &&
+      (m8(col_k) && m8(k_dim) && m8(k_nd) &&
        (k_rot0 < 0 || m8(k_rot0)) && m8(VW) && (col_v < 0 || m8(col_v)) &&
        (uintptr_t)k_cache % 16 == 0);
   if (bf && q_ok && k_ok && m8(ld_src) && (uintptr_t)src % 16 == 0 &&

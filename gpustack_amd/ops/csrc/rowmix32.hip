@@ -553,14 +553,14 @@ DEVICE_INLINE float act_fn(float z, int mode) {
 
 template <typename T>
 __global__ void act_and_mul_kernel(T* __restrict__ out, const T* __restrict__ gu,
-                                   long rows, int F, int mode) {
+                                   long ld_gu, long rows, int F, int mode) {
   const long n = rows * F;
   for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n;
        i += (long)gridDim.x * blockDim.x) {
     const long r = i / F;
     const int c = (int)(i % F);
-    const float g = ld(gu + r * 2 * F + c);
-    const float u = ld(gu + r * 2 * F + F + c);
+    const float g = ld(gu + r * ld_gu + c);
+    const float u = ld(gu + r * ld_gu + F + c);
     st(out + i, act_fn(g, mode) * u);
   }
 }
@@ -579,13 +579,13 @@ DEVICE_INLINE float act_fast(float z, int mode) {
 template <int MODE>
 __global__ __launch_bounds__(256) void act_and_mul_vec_kernel(
     unsigned short* __restrict__ out, const unsigned short* __restrict__ gu,
-    long rows, int F8) {
+    long ld8, long rows, int F8) {
   const long n = rows * F8;
   for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n;
        i += (long)gridDim.x * blockDim.x) {
     const long r = i / F8;
     const int c = (int)(i % F8);
-    const u16x8* gp = reinterpret_cast<const u16x8*>(gu) + r * 2 * F8 + c;
+    const u16x8* gp = reinterpret_cast<const u16x8*>(gu) + r * ld8 + c;
     const u16x8 g = gp[0], u = gp[F8];
     u16x8 o;
 #pragma unroll
@@ -710,28 +710,30 @@ void diff_combine_launch(void* out, const float* a, const float* lam,
         (float*)out, a, lam, diff, eps, n_heads, VW);
 }
 
-void act_and_mul_launch(void* out, const void* gu, long rows, int F, int mode,
-                        int bf, hipStream_t s) {
+// ld_gu: elements between two rows of gu (>= 2 F)
+void act_and_mul_launch(void* out, const void* gu, long ld_gu, long rows, int F,
+                        int mode, int bf, hipStream_t s) {
   const long n = rows * F;
   if (n <= 0) return;
-  if (bf && F % 8 == 0) {
+  if (bf && F % 8 == 0 && ld_gu % 8 == 0 && (uintptr_t)gu % 16 == 0) {
+    const long ld8 = ld_gu / 8;
     const long n8 = n / 8;
     const int g8 = (int)min((n8 + 255) / 256, (long)(256 * 64));
     auto* o = (unsigned short*)out;
     auto* g = (const unsigned short*)gu;
     switch (mode) {
-      case 0: act_and_mul_vec_kernel<0><<<g8, 256, 0, s>>>(o, g, rows, F / 8); break;
-      case 1: act_and_mul_vec_kernel<1><<<g8, 256, 0, s>>>(o, g, rows, F / 8); break;
-      case 2: act_and_mul_vec_kernel<2><<<g8, 256, 0, s>>>(o, g, rows, F / 8); break;
-      default: act_and_mul_vec_kernel<3><<<g8, 256, 0, s>>>(o, g, rows, F / 8); break;
+      case 0: act_and_mul_vec_kernel<0><<<g8, 256, 0, s>>>(o, g, ld8, rows, F / 8); break;
+      case 1: act_and_mul_vec_kernel<1><<<g8, 256, 0, s>>>(o, g, ld8, rows, F / 8); break;
+      case 2: act_and_mul_vec_kernel<2><<<g8, 256, 0, s>>>(o, g, ld8, rows, F / 8); break;
+      default: act_and_mul_vec_kernel<3><<<g8, 256, 0, s>>>(o, g, ld8, rows, F / 8); break;
     }
     return;
   }
   const int grid = (int)min((n + 255) / 256, (long)(256 * 32));
   if (bf)
     act_and_mul_kernel<unsigned short><<<grid, 256, 0, s>>>(
-        (unsigned short*)out, (const unsigned short*)gu, rows, F, mode);
+        (unsigned short*)out, (const unsigned short*)gu, ld_gu, rows, F, mode);
   else
     act_and_mul_kernel<float><<<grid, 256, 0, s>>>(
-        (float*)out, (const float*)gu, rows, F, mode);
+        (float*)out, (const float*)gu, ld_gu, rows, F, mode);
 }

@@ -1,6 +1,6 @@
 // Torch bindings for the layer-norm row kernels, the head-norm cache write,
-// scored routing (lnrows32.hip) and the recurrent mixers (state_scan.hip,
-// delta_scan.hip);
+// scored routing (lnrows32.hip), the recurrent mixers (state_scan.hip,
+// delta_scan.hip) and the short convolution (short_conv.hip);
 // page-wise value stores come from rowmix32.hip. Every shape a kernel or its
 // grid assumes is checked here on the host before the launch; VALUES inside
 // index tensors are bounded in the kernels.
@@ -13,13 +13,11 @@ void add_layer_norm_launch(float*, const void*, const float*, const float*, void
 void head_norm_store_launch(void*, void*, long, int, int, int, const float*, const float*, int, float, float, const int*, const void*, long, const float*, void*, void*, const long*, long, int, int, int, float, int, int, int, hipStream_t);
 void value_page_store_launch(const void*, long, int, void*, const long*, long, const int*, int, int, int, int, int, int, hipStream_t);
 void route_topk_launch(int*, float*, const float*, int, const float*, int, int, int, int, int, int, int, int, float, hipStream_t);
-void causal_conv_silu_launch(void*, const void*, long, int, int, int, const float*, const float*, void*, const int*, const int*, const int*, const int*, const int*, int, int, int, int, hipStream_t);
 int state_scan_launch(float*, const void*, long, int, int, int, const void*, long, int, int, int, int, int, int, const float*, const float*, const float*, const float*, float*, const int*, const int*, const int*, const int*, int, int, int, int, int, hipStream_t);
 void gated_group_norm_launch(void*, const float*, const void*, long, const float*, int, int, int, float, int, int, int, hipStream_t);
 int delta_scan_launch(float*, const void*, long, int, int, int, const void*, long, int, int, int, int, int, int, const float*, const float*, float*, const int*, const int*, const int*, const int*, int, int, int, int, int, hipStream_t);
 int delta_scan_max_state();
 int state_scan_max_state();
-int conv_max_taps();
 
 #define HIP_CHECK_LAST()                                                     \
   do {                                                                       \
@@ -211,36 +209,6 @@ int seq_view(const Tensor& seq_first, const Tensor& seq_rows,
   return nseq;
 }
 
-void causal_conv_silu(Tensor out, Tensor src, long col0, Tensor w, Tensor b,
-                      Tensor conv_state, Tensor seq_first, Tensor seq_rows,
-                      Tensor state_slots, Tensor row_seq, Tensor pos32) {
-  const int bf = act_kind(out, "out");
-  TORCH_CHECK(view_kind(src, "src") == bf &&
-              act_kind(conv_state, "conv_state") == bf,
-              "out, src and the state must share a dtype");
-  chk(w, "w", at::kFloat);
-  chk(b, "b", at::kFloat);
-  chk(row_seq, "row_seq", at::kInt);
-  TORCH_CHECK(out.dim() == 2 && w.dim() == 2 && conv_state.dim() == 3);
-  const int T = out.size(0), C = out.size(1), taps = w.size(1);
-  TORCH_CHECK(src.size(0) == T && col0 >= 0 && col0 + C <= src.size(1));
-  TORCH_CHECK(w.size(0) == C && b.numel() == C && taps >= 1 &&
-              taps <= conv_max_taps());
-  TORCH_CHECK(taps == 1 || (conv_state.size(1) == taps - 1 &&
-                            conv_state.size(2) == C && conv_state.size(0) >= 1),
-              "state must be [slots, taps - 1, channels]");
-  const int nseq = seq_view(seq_first, seq_rows, state_slots, pos32, T);
-  TORCH_CHECK(row_seq.numel() == T);
-  causal_conv_silu_launch(out.data_ptr(), src.data_ptr(), src.stride(0),
-                          (int)col0, C, taps, w.data_ptr<float>(),
-                          b.data_ptr<float>(), conv_state.data_ptr(),
-                          seq_first.data_ptr<int>(), seq_rows.data_ptr<int>(),
-                          state_slots.data_ptr<int>(), row_seq.data_ptr<int>(),
-                          pos32.data_ptr<int>(), nseq, (int)conv_state.size(0),
-                          T, bf, cur_stream(src));
-  HIP_CHECK_LAST();
-}
-
 void state_scan(Tensor y, Tensor src, long col_x, long col_b, long col_c,
                 OptTensor dt_src, long col_dt, long heads, long groups,
                 long n_state, long vdim, bool act_silu, OptTensor dt_bias,
@@ -358,12 +326,14 @@ void gated_group_norm(Tensor out, Tensor y, Tensor gate, Tensor w, long groups,
 
 }  // namespace
 
+#include "short_conv_binding.h"
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("embed_rows_scaled", &embed_rows_scaled);
   m.def("add_layer_norm", &add_layer_norm);
   m.def("head_norm_store", &head_norm_store);
   m.def("route_topk", &route_topk);
-  m.def("causal_conv_silu", &causal_conv_silu);
+  m.def("short_conv", &short_conv);
   m.def("state_scan", &state_scan);
   m.def("delta_scan", &delta_scan);
   m.def("gated_group_norm", &gated_group_norm);

@@ -10,10 +10,6 @@
 // rows through that per-sequence view, so a prompt cut anywhere, a decode
 // row and a mixed batch give the same states.
 //
-//   causal_conv_silu : short causal convolution per channel + SiLU; the
-//                      inputs before this step's rows come from the slot's
-//                      last taps - 1 inputs; a second launch moves the
-//                      slot on (it must not race with the reads)
 //   state_scan       : the recurrence. A wave owns PL value channels of one
 //                      (sequence, head); the N state rows are split over
 //                      TPP lanes per channel, NR rows each, in registers.
@@ -43,122 +39,6 @@ DEVICE_INLINE float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 // softplus without a switch-over: max(x, 0) + log1p(exp(-|x|))
 DEVICE_INLINE float softplus_f(float x) {
   return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)));
-}
-
-constexpr int MAX_TAPS = 16;
-
-// grid (T, ceil(C / 256)): one lane per (row, channel).
-template <typename TS>
-__global__ __launch_bounds__(256) void causal_conv_silu_kernel(
-    TS* __restrict__ out, const TS* __restrict__ src, long ld_src, int col0,
-    int C, int taps, const float* __restrict__ w, const float* __restrict__ b,
-    const TS* __restrict__ conv_state, const int* __restrict__ seq_first,
-    const int* __restrict__ state_slots, const int* __restrict__ row_seq,
-    const int* __restrict__ pos32, int nseq, int nslots, int T) {
-  const int t = blockIdx.x;
-  const int c = blockIdx.y * 256 + threadIdx.x;
-  if (c >= C) return;
-  const int s = min(max(row_seq[t], 0), nseq - 1);
-  const int first = min(max(seq_first[s], 0), t);
-  const int i = t - first;                   // row index inside the portion
-  const int pos = max(pos32[t], 0);
-  const int slot = min(max(state_slots[s], 0), nslots - 1);
-  const int keep = taps - 1;
-  const TS* stp = conv_state + (long)slot * keep * C;
-  float acc = b[c];
-  for (int k = 0; k < taps; ++k) {
-    const int d = keep - k;                  // how far back this tap looks
-    float v = 0.f;
-    if (i - d >= 0)
-      v = ld(src + (long)(t - d) * ld_src + col0 + c);
-    else if (pos - d >= 0)
-      v = ld(stp + (long)(keep + i - d) * C + c);
-    acc += w[(long)c * taps + k] * v;
-  }
-  st(out + (long)t * C + c, silu_f(acc));
-}
-
-// The same for bf16 rows whose channel count, first column and row stride
-// are multiples of 8: a lane takes 8 neighbouring channels of RB rows in a
-// row with 16-byte loads, its TAPS x 8 weights in registers.
-// grid (ceil(T / RB), ceil(C / 8 / 256)).
-constexpr int RB = 8;
-
-template <int TAPS>
-__global__ __launch_bounds__(256) void causal_conv_silu_vec_kernel(
-    unsigned short* __restrict__ out, const unsigned short* __restrict__ src,
-    long ld_src, int col0, int C, const float* __restrict__ w,
-    const float* __restrict__ b, const unsigned short* __restrict__ conv_state,
-    const int* __restrict__ seq_first, const int* __restrict__ state_slots,
-    const int* __restrict__ row_seq, const int* __restrict__ pos32, int nseq,
-    int nslots, int T) {
-  const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
-  if (c >= C) return;
-  constexpr int keep = TAPS - 1;
-  float wr[TAPS][8], br[8];
-#pragma unroll
-  for (int e = 0; e < 8; ++e) {
-    br[e] = b[c + e];
-#pragma unroll
-    for (int k = 0; k < TAPS; ++k) wr[k][e] = w[(long)(c + e) * TAPS + k];
-  }
-  const int t_end = min(T, (int)(blockIdx.x + 1) * RB);
-  for (int t = blockIdx.x * RB; t < t_end; ++t) {
-    const int s = min(max(row_seq[t], 0), nseq - 1);
-    const int first = min(max(seq_first[s], 0), t);
-    const int i = t - first;
-    const int pos = max(pos32[t], 0);
-    const int slot = min(max(state_slots[s], 0), nslots - 1);
-    const unsigned short* stp = conv_state + (long)slot * keep * C;
-    float acc[8];
-#pragma unroll
-    for (int e = 0; e < 8; ++e) acc[e] = br[e];
-#pragma unroll
-    for (int k = 0; k < TAPS; ++k) {
-      const int d = keep - k;
-      u16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
-      if (i - d >= 0)
-        v = *reinterpret_cast<const u16x8*>(src + (long)(t - d) * ld_src + col0 + c);
-      else if (pos - d >= 0)
-        v = *reinterpret_cast<const u16x8*>(stp + (long)(keep + i - d) * C + c);
-#pragma unroll
-      for (int e = 0; e < 8; ++e) acc[e] += wr[k][e] * bf2f(v[e]);
-    }
-    u16x8 o;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) o[e] = f2bf(silu_f(acc[e]));
-    *reinterpret_cast<u16x8*>(out + (long)t * C + c) = o;
-  }
-}
-
-// grid (nseq, ceil(C / 256)): the slot's new last inputs, after every read
-// of the old ones (stream order).
-template <typename TS>
-__global__ __launch_bounds__(256) void conv_state_update_kernel(
-    const TS* __restrict__ src, long ld_src, int col0, int C, int taps,
-    TS* __restrict__ conv_state, const int* __restrict__ seq_first,
-    const int* __restrict__ seq_rows, const int* __restrict__ state_slots,
-    const int* __restrict__ pos32, int nslots, int T) {
-  const int s = blockIdx.x;
-  const int c = blockIdx.y * 256 + threadIdx.x;
-  if (c >= C) return;
-  const int first = seq_first[s], n = seq_rows[s];
-  if (first < 0 || n < 1 || first + n > T) return;
-  const int hist = max(pos32[first], 0);
-  const int slot = min(max(state_slots[s], 0), nslots - 1);
-  const int keep = taps - 1;
-  TS* stp = conv_state + (long)slot * keep * C;
-  TS fresh[MAX_TAPS];
-  for (int j = 0; j < keep; ++j) {
-    const int i = n - (keep - j);            // local row of new entry j
-    TS v = 0;
-    if (i >= 0)
-      v = src[(long)(first + i) * ld_src + col0 + c];
-    else if (hist + i >= 0)
-      v = stp[(long)(keep + i) * C + c];
-    fresh[j] = v;
-  }
-  for (int j = 0; j < keep; ++j) stp[(long)j * C + c] = fresh[j];
 }
 
 struct ScanArgs {
@@ -705,51 +585,6 @@ bool scan_pick(float* y, const void* src, const void* dt, const ScanArgs& p,
 }  // namespace
 
 int state_scan_max_state() { return 8 * 64; }
-int conv_max_taps() { return MAX_TAPS; }
-
-void causal_conv_silu_launch(void* out, const void* src, long ld_src, int col0,
-                             int C, int taps, const float* w, const float* b,
-                             void* conv_state, const int* seq_first,
-                             const int* seq_rows, const int* state_slots,
-                             const int* row_seq, const int* pos32, int nseq,
-                             int nslots, int T, int bf, hipStream_t s) {
-  if (T <= 0 || nseq <= 0) return;
-  dim3 grid(T, (C + 255) / 256), sgrid(nseq, (C + 255) / 256);
-  if (bf) {
-    // few rows (decode): one lane per (row, channel) makes more workgroups
-    const bool vec = C % 8 == 0 && col0 % 8 == 0 && ld_src % 8 == 0 &&
-                     (long)T * C >= (1 << 20);
-    const dim3 vgrid((T + RB - 1) / RB, (C / 8 + 255) / 256);
-#define CONV_VEC(TAPSV)                                                        \
-  causal_conv_silu_vec_kernel<TAPSV><<<vgrid, 256, 0, s>>>(                    \
-      (unsigned short*)out, (const unsigned short*)src, ld_src, col0, C, w, b, \
-      (const unsigned short*)conv_state, seq_first, state_slots, row_seq,      \
-      pos32, nseq, nslots, T)
-    if (vec && taps == 4) CONV_VEC(4);
-    else if (vec && taps == 3) CONV_VEC(3);
-    else if (vec && taps == 2) CONV_VEC(2);
-#undef CONV_VEC
-    else
-      causal_conv_silu_kernel<unsigned short><<<grid, 256, 0, s>>>(
-          (unsigned short*)out, (const unsigned short*)src, ld_src, col0, C,
-          taps, w, b, (const unsigned short*)conv_state, seq_first, state_slots,
-          row_seq, pos32, nseq, nslots, T);
-    if (taps > 1)
-      conv_state_update_kernel<unsigned short><<<sgrid, 256, 0, s>>>(
-          (const unsigned short*)src, ld_src, col0, C, taps,
-          (unsigned short*)conv_state, seq_first, seq_rows, state_slots, pos32,
-          nslots, T);
-  } else {
-    causal_conv_silu_kernel<float><<<grid, 256, 0, s>>>(
-        (float*)out, (const float*)src, ld_src, col0, C, taps, w, b,
-        (const float*)conv_state, seq_first, state_slots, row_seq, pos32, nseq,
-        nslots, T);
-    if (taps > 1)
-      conv_state_update_kernel<float><<<sgrid, 256, 0, s>>>(
-          (const float*)src, ld_src, col0, C, taps, (float*)conv_state,
-          seq_first, seq_rows, state_slots, pos32, nslots, T);
-  }
-}
 
 // src_bf: src and dt_src are bf16 (else fp32). single: the caller expects
 // one row per sequence (a hint: any batch is still computed correctly).

@@ -542,7 +542,8 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
                     keep_first: int = 0,
                     sinks: torch.Tensor | None = None,
                     slopes: torch.Tensor | None = None,
-                    softcap: float = 0.0) -> None:
+                    softcap: float = 0.0, chunk: int = 0,
+                    gate: torch.Tensor | None = None) -> None:
     """out[t, a] = softmax_j(scale * q[t, a] . k_j) . V over the visible
     keys j of row t's sequence: j <= pos(t), and with window > 0 also
     (pos(t) - j < window or j < keep_first). q: [T, A, D] with A = heads *
@@ -551,7 +552,9 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
     values. sinks (per head, or None) add exp(sink) to the denominator;
     slopes (per head, or None) take slope * (pos(t) - j) off the scaled
     score; softcap > 0 turns a scaled score s into softcap * tanh(s /
-    softcap) first."""
+    softcap) first. chunk > 0: only keys of the row's own chunk of
+    positions, j >= pos(t) - pos(t) % chunk. gate [T, heads]: a head's
+    output is multiplied by sigmoid(gate)."""
     T, A, D = q.shape
     nb, G, BS, KW = k_cache.shape
     VW = v_cache.shape[2]
@@ -563,6 +566,8 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
         j = torch.arange(p + 1, device=q.device)
         if window > 0:
             j = j[(p - j < window) | (j < keep_first)]
+        if chunk > 0:
+            j = j[j >= p - p % chunk]
         blk = bt[j // BS].long()
         K = k_cache[blk, :, j % BS].float()                  # [L, G, KW]
         V = v_cache[blk, :, :, j % BS].float()               # [L, G, VW]
@@ -581,7 +586,10 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
             den = e.sum()
             if sinks is not None:
                 den = den + torch.exp(sinks[a // maps].float() - mx)
-            out[t, a] = ((e / den) @ V[:, g]).to(out.dtype)
+            o = (e / den) @ V[:, g]
+            if gate is not None:
+                o = o * torch.sigmoid(gate[t, a // maps].float())
+            out[t, a] = o.to(out.dtype)
 
 
 def diff_combine(out: torch.Tensor, a: torch.Tensor, lam: torch.Tensor,
@@ -666,12 +674,13 @@ def head_norm_store(q_out: torch.Tensor, qkv: torch.Tensor, nq: int, nk: int,
     v_cache[blk, :, :, off] = v[ok]
 
 
-def causal_conv_silu(out: torch.Tensor, src: torch.Tensor, col0: int,
-                     w: torch.Tensor, b: torch.Tensor,
-                     conv_state: torch.Tensor, seq_first: torch.Tensor,
-                     seq_rows: torch.Tensor, state_slots: torch.Tensor,
-                     pos32: torch.Tensor) -> None:
-    """out[t, c] = silu(b[c] + sum_k w[c, k] * in_c(t - (taps - 1 - k)))
+def short_conv(out: torch.Tensor, src: torch.Tensor, col0: int,
+               w: torch.Tensor, b: torch.Tensor | None,
+               conv_state: torch.Tensor | None, seq_first: torch.Tensor,
+               seq_rows: torch.Tensor, state_slots: torch.Tensor,
+               pos32: torch.Tensor, silu: bool = True) -> None:
+    """out[t, c] = act(b[c] + sum_k w[c, k] * in_c(t - (taps - 1 - k))), act
+    SiLU or nothing,
     per channel c of src[:, col0:col0 + C], within each sequence; inputs
     before this step's rows come from conv_state[slot] (the sequence's last
     taps - 1 inputs, oldest first), inputs before position 0 are zero. The
@@ -691,10 +700,14 @@ def causal_conv_silu(out: torch.Tensor, src: torch.Tensor, col0: int,
             full = torch.cat([old, x], 0)
         else:
             full = x
-        acc = b.float()[None, :].repeat(n, 1)
+        acc = torch.zeros(n, C, device=src.device)
+        if b is not None:
+            acc = acc + b.float()[None, :]
         for k in range(taps):
             acc = acc + full[k:k + n] * w[:, k].float()[None, :]
-        out[r0:r0 + n] = (acc * torch.sigmoid(acc)).to(out.dtype)
+        if silu:
+            acc = acc * torch.sigmoid(acc)
+        out[r0:r0 + n] = acc.to(out.dtype)
         if keep:
             conv_state[slot] = full[full.shape[0] - keep:].to(conv_state.dtype)
 
@@ -818,8 +831,8 @@ def head_rope_store(q_out: torch.Tensor | None, src: torch.Tensor, col_q: int,
     """Row kernel between a projection and attention. The q side: q_heads
     heads of q_dim channels at src[:, col_q:]; the k side: k_heads heads of
     k_dim channels at src[:, col_k:] (k_heads 0: none). Per head, in fp32:
-    the first *_norm_dims channels are RMS-normed over themselves and
-    multiplied by *_w (None: no norm); then the 2 * len(inv_freq) channels
+    the first *_norm_dims channels (0: no norm) are RMS-normed over
+    themselves and multiplied by *_w (None: by nothing); then the 2 * len(inv_freq) channels
     from *_rot0 on turn by pos * f (rot0 < 0: no rotation) — channel i with
     i + half (half_layout) or 2i with 2i+1 — with cos and sin multiplied by
     `amplitude`. q heads go to q_out [T, q_heads * q_dim]; k heads to their
@@ -834,10 +847,10 @@ def head_rope_store(q_out: torch.Tensor | None, src: torch.Tensor, col_q: int,
 
     def prep(col, heads, dim, w, nd, rot0):
         t = src[:, col:col + heads * dim].float().reshape(T, heads, dim).clone()
-        if w is not None:
+        if nd > 0:
             part = t[..., :nd]
-            t[..., :nd] = part * torch.rsqrt(
-                part.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+            part = part * torch.rsqrt(part.pow(2).mean(-1, keepdim=True) + eps)
+            t[..., :nd] = part if w is None else part * w.float()
         if rot0 >= 0 and half:
             r = t[..., rot0:rot0 + 2 * half]
             if half_layout:
@@ -934,3 +947,81 @@ def head_gate(out: torch.Tensor, o_hts: torch.Tensor, gate_src: torch.Tensor,
     g = torch.sigmoid(gate_src[:, col:col + H].float())          # [T, H]
     o = o_hts.float().transpose(0, 1) * g[:, :, None]
     out.copy_(o.reshape(T, H * VD).to(out.dtype))
+
+
+# --- parallel residual streams, token shift, gated recurrence --------------
+
+def embed_streams(x: torch.Tensor, tokens: torch.Tensor, embed: torch.Tensor,
+                  scale: float) -> None:
+    """x[t, s] = embed[token_t] * scale for every stream s; x [T, S, W] fp32."""
+    x.copy_((embed[tokens].float() * scale)[:, None, :].expand_as(x))
+
+
+def stream_step(x: torch.Tensor, a: torch.Tensor | None,
+                gate: torch.Tensor | None, gate_b: torch.Tensor | None,
+                mix: torch.Tensor | None, out_w: torch.Tensor | None,
+                in_w: torch.Tensor | None, norm_w: torch.Tensor | None,
+                eps: float, h: torch.Tensor | None) -> None:
+    """Close one sublayer on the fp32 streams x [T, S, W] and open the next:
+        y = a * sigmoid(gate + gate_b)
+        x_t <- sum_s mix[s, t] x_s + out_w[t] y       (all from the old ones)
+        u = sum_s in_w[s] x_s;   h = rmsnorm(u) * norm_w   in h's dtype
+    a None: nothing to close; in_w None: nothing to open."""
+    if a is not None:
+        y = a.float()
+        if gate is not None:
+            g = gate.float()
+            if gate_b is not None:
+                g = g + gate_b.float()
+            y = y * torch.sigmoid(g)
+        new = torch.einsum("st,nsw->ntw", mix.float(), x) \
+            + out_w.float()[None, :, None] * y[:, None, :]
+        x.copy_(new)
+    if in_w is not None:
+        u = torch.einsum("s,nsw->nw", in_w.float(), x)
+        n = u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eps)
+        h.copy_((n * norm_w.float()).to(h.dtype))
+
+
+def token_shift(hs: torch.Tensor, h: torch.Tensor, mu: torch.Tensor,
+                state: torch.Tensor, seq_first: torch.Tensor,
+                seq_rows: torch.Tensor, state_slots: torch.Tensor,
+                pos32: torch.Tensor) -> None:
+    """hs[t] = h[t] + (h_prev - h[t]) * mu with h_prev the row before in the
+    same sequence; the row before this step's first one is state[slot] (zero
+    at position 0). The state then holds the step's last row of h."""
+    for s in range(seq_first.numel()):
+        r0, n, slot = int(seq_first[s]), int(seq_rows[s]), int(state_slots[s])
+        x = h[r0:r0 + n].float()
+        first = state[slot].float()[None] if int(pos32[r0]) > 0 \
+            else torch.zeros_like(x[:1])
+        prev = torch.cat([first, x[:-1]], 0)
+        hs[r0:r0 + n] = (x + (prev - x) * mu.float()).to(hs.dtype)
+        state[slot] = h[r0 + n - 1].to(state.dtype)
+
+
+def gru_scan(y: torch.Tensor, src: torch.Tensor, col_z: int, col_u: int,
+             col_g: int, z_b: torch.Tensor, u_b: torch.Tensor,
+             state: torch.Tensor, seq_first: torch.Tensor,
+             seq_rows: torch.Tensor, state_slots: torch.Tensor,
+             pos32: torch.Tensor) -> None:
+    """Per channel and sequence, over this step's rows in order, in fp32:
+        z = sigmoid(src[t, col_z + c] + z_b);  u = src[t, col_u + c] + u_b
+        S <- (1 - z) S + z * (u + 1/2 if u >= 0 else sigmoid(u))
+        y[t, c] = S * silu(src[t, col_g + c])
+    S is read from state[slot] (zero when the first row sits at position 0)
+    and written back; state [slots, ..., N] fp32."""
+    N = y.shape[1]
+    st = state.view(state.shape[0], N)
+    z = torch.sigmoid(src[:, col_z:col_z + N].float() + z_b.float())
+    u = src[:, col_u:col_u + N].float() + u_b.float()
+    c = torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+    g = src[:, col_g:col_g + N].float()
+    g = g * torch.sigmoid(g)
+    for s in range(seq_first.numel()):
+        r0, n, slot = int(seq_first[s]), int(seq_rows[s]), int(state_slots[s])
+        S = st[slot].clone() if int(pos32[r0]) > 0 else torch.zeros_like(st[slot])
+        for t in range(r0, r0 + n):
+            S = (1.0 - z[t]) * S + z[t] * c[t]
+            y[t] = (S * g[t]).to(y.dtype)
+        st[slot] = S
