@@ -94,15 +94,16 @@ def sees(i, j, chunk):
     return j <= i and (chunk <= 0 or i // chunk == j // chunk)
 
 
-def attend(q, k, v, scale, chunk=0, one_in_denominator=False):
+def attend(q, k, v, scale, chunk=0, one_in_denominator=False, misplaced=0):
     """One head: q, k [T, D], v [T, VD]. chunk > 0: keys of the query's own
-    chunk of positions only. one_in_denominator: exp(0) joins the sum."""
+    chunk of positions only. one_in_denominator: exp(0) joins the sum.
+    misplaced: a planted mistake, chunk borders that many positions off."""
     T = q.shape[0]
     i, j = torch.arange(T)[:, None], torch.arange(T)[None, :]
     mask = j <= i
     if chunk > 0:
-        mask = mask & (i // chunk == j // chunk)
-    if T <= 8:      # the table above is `sees`, element by element
+        mask = mask & ((i + misplaced) // chunk == (j + misplaced) // chunk)
+    if T <= 8 and not misplaced:      # the table above is `sees`, element by element
         assert all(bool(mask[a, b]) == sees(a, b, chunk)
                    for a in range(T) for b in range(T))
     s = ((q @ k.t()) * scale).masked_fill(~mask, -float("inf"))
@@ -134,15 +135,16 @@ def attention_mixer(h, m, w, p, eps, kind):
     rot = m["rot"]
     q = rotate(q, float(rot["base"]), int(rot["dims"]))
     k = rotate(k, float(rot["base"]), int(rot["dims"]))
-    chunk, one = 0, False
+    chunk, one, off = 0, False, 0
     if kind == "attention":
         q, k = rms_unit(q, eps), rms_unit(k, eps)
     else:
-        chunk, one = int(m["mask"]["size"]), True
+        chunk, one = int(m["mask"]["size"]), not m["mask"].get("no_one")
+        off = int(m["mask"].get("misplaced", 0))
     gate = torch.sigmoid(h @ W("g").t())                         # [T, H]
     rep = H // G
     outs = [attend(q[a], k[a // rep], v[a // rep], float(m["scale"]), chunk,
-                   one) * gate[:, a:a + 1] for a in range(H)]
+                   one, off) * gate[:, a:a + 1] for a in range(H)]
     return torch.cat(outs, -1) @ W("o").t()
 
 
