@@ -1,5 +1,5 @@
-"""Layer-level comparison bench: a Vunitar, Fusipel, Livasun or Makezen stack (`family`) at
-real-model layer sizes beside the closest llama-lineage stack of equal
+"""Layer-level comparison bench: a Vunitar, Fusipel, Livasun, Makezen or
+Fuvuvik stack (`family`) at real-model layer sizes beside the closest llama-lineage stack of equal
 width, depth and heads (random weights, synthetic tokens). Reports end-to-end prefill and decode
 throughput through LLMEngine for both, and per-kernel rates of the new
 kernels next to their counterparts with the fraction of the MI355X
@@ -161,6 +161,35 @@ def makezen_spec(s, moe: bool = False):
 
 def makezen_rank(s) -> int:
     return 256 if s["width"] <= 1024 else 384
+
+
+def fuvuvik_spec(s, moe: bool = False):
+    """Layers cycle chunked attention (head size 128, heads/4 kv heads,
+    chunks of 1024, one more in the denominator), causal attention behind a
+    4-tap convolution with unit q / k heads, and two gated recurrences of
+    the model width, on 4 residual streams; 64 rotated channels, head gates,
+    gated tanh-GELU feed-forward of the llama stack's width."""
+    from ..engine.config import (FeedForwardSpec, GruMixerSpec, LayerSpec,
+                                 ModelSpec, PagedMixerSpec, RotarySpec)
+
+    H, W = s["heads"], s["width"]
+    att = dict(heads=H, kv_heads=max(1, H // 4), qk_dim=128, v_dim=128,
+               scale=128 ** -0.5, out_gate=True,
+               rot=RotarySpec(dims=64, base=10000.0, layout="half"))
+    ff = FeedForwardSpec(kind="dense", ff=s["ff"], act="gelu_tanh", gated=True)
+    gru = ("gru", GruMixerSpec(width=W))
+    cycle = [("paged_attention",
+              PagedMixerSpec(**att, chunk=1024, unit_sink=True)),
+             ("paged_attention",
+              PagedMixerSpec(**att, conv=4, unit_norm=True)), gru, gru]
+    return ModelSpec(
+        architecture="Fuvuvik", vocab_size=32000, hidden_size=W,
+        num_layers=s["layers"],
+        layers=tuple(LayerSpec(*cycle[i % 4], ff) for i in range(s["layers"])),
+        num_heads=1, num_kv_heads=1, head_dim=8, intermediate_size=0,
+        rms_norm_eps=1e-5, max_position_embeddings=1 << 20, eos_token_id=-1,
+        fp32_residual=True, streams=4, token_shift=True, residual_gate=True,
+        embed_scale=1.0)
 
 
 def llama_spec(s, moe: bool):
@@ -947,23 +976,195 @@ def makezen_kernel_rates(s, device):
     return out
 
 
+def fuvuvik_kernel_rates(s, device):
+    """Per-kernel rates of the Fuvuvik kernels next to their likes in the
+    Livasun stack (windowed attention, matrix-state scan and step, its row
+    kernels, the convolution with SiLU)."""
+    from .. import ops
+
+    bf = torch.bfloat16
+    H, W, D, BS, S = s["heads"], s["width"], 128, 16, 4
+    G = max(1, H // 4)
+    out = []
+
+    def rec(name, sec, flops=None, nbytes=None, peak=PEAK_FLOPS):
+        if flops is not None:
+            out.append(dict(kernel=name, us=round(sec * 1e6, 1),
+                            tflops=round(flops / sec / 1e12, 1),
+                            roofline=round(flops / sec / peak, 4)))
+        else:
+            out.append(dict(kernel=name, us=round(sec * 1e6, 1),
+                            gbps=round(nbytes / sec / 1e9, 1),
+                            roofline=round(nbytes / sec / PEAK_BW, 4)))
+
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=device)
+    zeros = torch.zeros(H, device=device)
+    slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / H) for h in range(H)],
+                          device=device)
+    # ---- prefill attention: 4 prompts x 2048; decode: 64 x 2048 cached ----
+    win = 1024
+    for phase, nseq, hist, L in (("prefill", 4, 0, 2048), ("decode", 64, 2047, 1)):
+        ctx, T = hist + L, nseq * L
+        nblk = nseq * (ctx // BS) + 1
+        bt = torch.arange(nseq * (ctx // BS), dtype=torch.int32,
+                          device=device).view(nseq, -1)
+        row_seq = torch.arange(nseq, dtype=torch.int32,
+                               device=device).repeat_interleave(L)
+        pos = torch.arange(hist, ctx, dtype=torch.int32, device=device).repeat(nseq)
+        kc = torch.randn(nblk, G, BS, D, device=device).to(bf)
+        vc = torch.randn(nblk, G, D, BS, device=device).to(bf)
+        qkvg = torch.randn(T, (H + 2 * G) * D + H, device=device).to(bf)
+        q = qkvg[:, :H * D].contiguous().view(T, H, D)
+        o = torch.empty_like(q)
+        gate = qkvg[:, -H:]
+        tiles = ops.build_attn_tiles([i * L for i in range(nseq)],
+                                     [hist] * nseq, [L] * nseq, H, G, 1, device)
+        for label, seen, kw in (
+                ("causal + head gates", lambda i: i + 1, dict(gate=gate)),
+                ("chunks of 1024 + unit sink + head gates",
+                 lambda i: i % win + 1,
+                 dict(chunk=win, sinks=zeros, gate=gate)),
+                ("window 1024 + slopes (Livasun)", lambda i: min(i + 1, win),
+                 dict(window=win, slopes=slopes))):
+            n = nseq * sum(seen(i) for i in range(hist, ctx))
+            sec = _time(lambda: ops.paged_attention(
+                o, q, kc, vc, bt, row_seq, pos, D ** -0.5, tiles=tiles,
+                max_ctx=ctx if L == 1 else 0, **kw), 5 if L > 1 else 20)
+            if L > 1:
+                rec(f"paged_attention {phase}, {label} (mfma, useful pairs)",
+                    sec, flops=4.0 * D * H * n)
+            else:
+                rec(f"paged_attention {phase}, {label} (mfma)", sec,
+                    nbytes=n * G * D * 4)
+
+    # ---- row kernels at T = 8192 rows, and 64 decode rows ----
+    w32, b32 = torch.ones(W, device=device), torch.zeros(W, device=device)
+    mix = torch.eye(S, device=device) * 0.9 + 0.02
+    rw = torch.full((S,), 1.0 / S, device=device)
+    nq, nk = H * D, G * D
+    wd = torch.ones(D, device=device)
+    inv = torch.tensor([10000.0 ** (-i / 32) for i in range(32)], device=device)
+    for T in (8192, 64):
+        lab = f"{T} rows"
+        x = torch.randn(T, S, W, device=device)
+        a = torch.randn(T, W, device=device).to(bf)
+        r = torch.randn(T, W, device=device).to(bf)
+        hb, hs = torch.empty_like(a), torch.empty_like(a)
+        state = torch.zeros(65, W, dtype=bf, device=device)
+        nseq = 8 if T > 64 else 64
+        L = T // nseq
+        sf, sr = i32([i * L for i in range(nseq)]), i32([L] * nseq)
+        ss = i32(list(range(nseq)))
+        rs = torch.arange(nseq, dtype=torch.int32, device=device).repeat_interleave(L)
+        p32 = (torch.arange(L, dtype=torch.int32, device=device) + 5).repeat(nseq)
+        shift = (hs, w32, state, rs, ss, p32) if L == 1 else None
+        rec(f"stream_step (gate, 4 streams mixed, norm{', shift' if shift else ''}), {lab}",
+            _time(lambda: ops.stream_step(x, a, r, b32, mix, rw, rw, w32, 1e-5,
+                                          hb, shift=shift)),
+            nbytes=T * W * (8 * S + 6 + (6 if shift else 0)))
+        if not shift:
+            rec(f"token_shift, {lab}",
+                _time(lambda: ops.token_shift(hs, hb, w32, state, sf, sr, ss,
+                                              rs, p32)), nbytes=T * W * 4)
+        x1 = torch.randn(T, W, device=device)
+        rec(f"add_layer_norm (Livasun: add + layer norm), {lab}",
+            _time(lambda: ops.add_layer_norm(x1, a, w32, w32, 1e-5, hb)),
+            nbytes=T * W * 12)
+        nblk = T // BS + 1
+        kc = torch.zeros(nblk, G, BS, D, dtype=bf, device=device)
+        vc = torch.zeros(nblk, G, D, BS, dtype=bf, device=device)
+        C = nq + 2 * nk
+        u = torch.randn(T, C + H, device=device).to(bf)
+        qkv = torch.empty(T, C, dtype=bf, device=device)
+        qo = torch.empty(T, nq, dtype=bf, device=device)
+        slots = torch.arange(T, device=device)
+        pg = ops.build_page_groups([0], [0], [T], BS, device) if L > 1 else None
+        nb_rows = T * (2 * nq + 4 * nk) * 2
+        cw, cb = torch.randn(C, 4, device=device), torch.zeros(C, device=device)
+        cst = torch.zeros(nseq + 1, 3, C, dtype=bf, device=device)
+        rec(f"short_conv (q | k | v), {lab}",
+            _time(lambda: ops.short_conv(qkv, u, 0, cw, None, cst, sf, sr, ss,
+                                         rs, p32, silu=False, single=L == 1)),
+            nbytes=T * C * 4)
+        rec(f"causal_conv_silu (Livasun), {lab}",
+            _time(lambda: ops.causal_conv_silu(qkv, u, 0, cw, cb, cst, sf, sr,
+                                               ss, rs, p32)), nbytes=T * C * 4)
+        rec(f"head_rope_store, unit heads + rotation + cache write, {lab}",
+            _time(lambda: ops.head_rope_store(
+                qo, qkv, 0, H, D, None, D, 0, nq, G, D, None, D, 0, nq + nk,
+                inv, True, 1.0, p32, kc, vc, slots, 1e-5, page_groups=pg)),
+            nbytes=nb_rows)
+        vfirst = torch.randn(T, nk, device=device).to(bf)
+        lam = torch.tensor([0.3], device=device)
+        rec(f"head_norm_store (Livasun: head norms + temperature + blend + cache write), {lab}",
+            _time(lambda: ops.head_norm_store(qo, qkv, nq, nk, wd, wd, D, 0.1,
+                                              1024, p32, vfirst, lam, kc, vc,
+                                              slots, 1e-5, page_groups=pg)),
+            nbytes=nb_rows + T * nk * 2)
+        gu = torch.randn(T, 2 * s["ff"] + W, device=device).to(bf)
+        gc = gu[:, :2 * s["ff"]].contiguous()
+        ao = torch.empty(T, s["ff"], dtype=bf, device=device)
+        rec(f"act_and_mul gelu_tanh, strided rows, {lab}",
+            _time(lambda: ops.act_and_mul(ao, gu[:, :2 * s["ff"]], "gelu_tanh")),
+            nbytes=T * s["ff"] * 6)
+        rec(f"act_and_mul silu (Livasun), {lab}",
+            _time(lambda: ops.act_and_mul(ao, gc, "silu")),
+            nbytes=T * s["ff"] * 6)
+
+    # ---- recurrences ----
+    for label, nseq, L in (("prefill 8 x 1024", 8, 1024),
+                           ("prefill 1 x 8192", 1, 8192),
+                           ("decode 64 x 1", 64, 1)):
+        T = nseq * L
+        starts = [i * L for i in range(nseq)]
+        sf, sr = i32(starts), i32([L] * nseq)
+        ss = i32(list(range(nseq)))
+        ps = (torch.arange(L, dtype=torch.int32, device=device) + 5).repeat(nseq)
+        u = torch.randn(T, 3 * W, device=device).to(bf)
+        yb = torch.empty(T, W, dtype=bf, device=device)
+        st = torch.zeros(nseq + 1, 1, 1, W, device=device)
+        ch = ops.build_scan_chunks(starts, [L] * nseq, ops.SCAN_CHUNK, device) \
+            if L > ops.SCAN_CHUNK else None
+        rec(f"gru_scan {label}",
+            _time(lambda: ops.gru_scan(yb, u, 0, W, 2 * W, b32, b32, st, sf, sr,
+                                       ss, ps, chunks=ch)),
+            nbytes=T * W * 8 + nseq * W * 8)
+        y = torch.empty(T, H * 128, device=device)
+        ul = torch.randn(T, 4 * H * 128, device=device).to(bf)
+        stl = torch.zeros(nseq + 1, H, 128, 128, device=device)
+        dec = torch.full((H,), 0.99, device=device)
+        sec = _time(lambda: ops.state_scan(y, ul, 2 * H * 128, H * 128, 0, None,
+                                           0, H, H, 128, 128, True, None, None,
+                                           None, dec, stl, sf, sr, ss, ps,
+                                           single=L == 1), 5)
+        if L > 1:
+            rec(f"state_scan lightning {label} (Livasun, 4 flops per state element)",
+                sec, flops=4.0 * T * H * 128 * 128, peak=PEAK_VALU)
+        else:
+            rec(f"state_scan lightning {label} (Livasun, state read + write)",
+                sec, nbytes=nseq * H * 128 * 128 * 8)
+    return out
+
+
 def run(sizes: list[str], device: str, family: str = "vunitar",
         solo: bool = False) -> None:
     """`solo`: only the family's own stack end to end (no comparison stack,
     no per-kernel rates) — the run to put under a profiler."""
     for name in sizes:
         s = SIZES[name]
-        if family in ("livasun", "makezen"):
+        if family in ("livasun", "makezen", "fuvuvik"):
             s = dict(s, layers=4)       # one full cycle of the mixers
         for moe in ((False, True) if family in ("vunitar", "livasun")
                     else (False,)):
             row = {"size": name, **s, "ff_kind": "moe" if moe else "dense"}
             mine = {"vunitar": vunitar_spec, "fusipel": fusipel_spec,
-                    "livasun": livasun_spec, "makezen": makezen_spec}[family]
-            # Makezen's closest existing model is the other hybrid of
-            # attention and recurrent layers; the llama graph for scale
-            others = ((("livasun", livasun_spec),) if family == "makezen"
-                      else ()) + (("llama_graph", llama_spec),)
+                    "livasun": livasun_spec, "makezen": makezen_spec,
+                    "fuvuvik": fuvuvik_spec}[family]
+            # Makezen's and Fuvuvik's closest existing model is another
+            # hybrid of attention and recurrent layers; the llama graph for
+            # scale
+            others = ((("livasun", livasun_spec),)
+                      if family in ("makezen", "fuvuvik") else ()) + (("llama_graph", llama_spec),)
             for label, mk in ((family, mine),) + (() if solo else others):
                 pre, dec = engine_rates(mk(s, moe), device)
                 row[label] = {"prefill_tok_s": round(pre), "decode_tok_s": round(dec)}
@@ -971,6 +1172,7 @@ def run(sizes: list[str], device: str, family: str = "vunitar",
         if torch.cuda.is_available() and not solo:
             rates = {"vunitar": kernel_rates, "fusipel": fusipel_kernel_rates,
                      "livasun": livasun_kernel_rates,
-                     "makezen": makezen_kernel_rates}[family]
+                     "makezen": makezen_kernel_rates,
+                     "fuvuvik": fuvuvik_kernel_rates}[family]
             for k in rates(s, device):
                 print(json.dumps({"kernel_bench": {"size": name, **k}}), flush=True)

@@ -31,7 +31,11 @@ template <> DEVICE_INLINE void st<unsigned short>(unsigned short* p, float v) {
   *p = f2bf(v);
 }
 
-DEVICE_INLINE float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+// hardware exponential and reciprocal, each within a few ulp of fp32; an
+// overflowing exponential gives rcp(inf) = 0
+DEVICE_INLINE float sigmoid_f(float z) {
+  return __builtin_amdgcn_rcpf(1.0f + __expf(-z));
+}
 DEVICE_INLINE float candidate(float u) {
   return u >= 0.f ? u + 0.5f : sigmoid_f(u);
 }

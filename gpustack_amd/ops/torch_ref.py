@@ -680,8 +680,7 @@ def short_conv(out: torch.Tensor, src: torch.Tensor, col0: int,
                seq_rows: torch.Tensor, state_slots: torch.Tensor,
                pos32: torch.Tensor, silu: bool = True) -> None:
     """out[t, c] = act(b[c] + sum_k w[c, k] * in_c(t - (taps - 1 - k))), act
-    SiLU or nothing,
-    per channel c of src[:, col0:col0 + C], within each sequence; inputs
+    SiLU or nothing, per channel c of src[:, col0:col0 + C], within each sequence; inputs
     before this step's rows come from conv_state[slot] (the sequence's last
     taps - 1 inputs, oldest first), inputs before position 0 are zero. The
     state then takes the last taps - 1 inputs including this step's."""
@@ -710,6 +709,13 @@ def short_conv(out: torch.Tensor, src: torch.Tensor, col0: int,
         out[r0:r0 + n] = acc.to(out.dtype)
         if keep:
             conv_state[slot] = full[full.shape[0] - keep:].to(conv_state.dtype)
+
+
+def causal_conv_silu(out, src, col0, w, b, conv_state, seq_first, seq_rows,
+                     state_slots, pos32) -> None:
+    """short_conv with a bias and SiLU."""
+    short_conv(out, src, col0, w, b, conv_state, seq_first, seq_rows,
+               state_slots, pos32)
 
 
 def state_scan(y: torch.Tensor, src: torch.Tensor, col_x: int, col_b: int,

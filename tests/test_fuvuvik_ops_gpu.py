@@ -48,7 +48,7 @@ def test_stream_step(dtype, S, W, T):
     eps = 1e-5
     # gate rows of a wider product, at an aligned and an unaligned column
     for col in (8, 3):
-        gate = wide[:, col:col + W] if col == 8 else wide[:, col:col + W]
+        gate = wide[:, col:col + W]
         xr, hr = x.clone(), torch.zeros(T, W, dtype=dtype)
         torch_ref.stream_step(xr, a, gate, gb, mix, b, rd, nw, eps, hr)
         xg, hg = x.cuda(), torch.zeros(T, W, dtype=dtype, device="cuda")
