@@ -3,8 +3,8 @@
 //
 //   head_rope_store : per head of a q side and a k side of one projection
 //                     row: RMS norm of the head's first channels with or
-//                     without a weight vector shared by the heads, then rotation of a
-//                     channel range (pairs (i, i + half) or (2i, 2i + 1),
+//                     without a weight vector shared by the heads, then
+//                     rotation of a channel range (pairs (i, i + half) or (2i, 2i + 1),
 //                     cos / sin times an amplitude); q heads out, k heads
 //                     into their page rows, values into the transposed
 //                     value pages — from the projection, or the first

@@ -680,7 +680,8 @@ def short_conv(out: torch.Tensor, src: torch.Tensor, col0: int,
                seq_rows: torch.Tensor, state_slots: torch.Tensor,
                pos32: torch.Tensor, silu: bool = True) -> None:
     """out[t, c] = act(b[c] + sum_k w[c, k] * in_c(t - (taps - 1 - k))), act
-    SiLU or nothing, per channel c of src[:, col0:col0 + C], within each sequence; inputs
+    SiLU or nothing, per channel c of src[:, col0:col0 + C], within each
+    sequence; inputs
     before this step's rows come from conv_state[slot] (the sequence's last
     taps - 1 inputs, oldest first), inputs before position 0 are zero. The
     state then takes the last taps - 1 inputs including this step's."""
