@@ -203,7 +203,22 @@ class ScanMixerSpec:
       q, k (shared by the heads of a group) and v pass a causal convolution
       of `conv` taps and SiLU, then q and k are scaled to unit length (q
       also by state^(-1/2)); each head's output is RMS-normed, weighted and
-      multiplied by a SiLU gate."""
+      multiplied by a SiLU gate.
+    * kind "retention": a_t = decay[h] (constants), b_t = 1; q and k turn
+      with the position (`rot`), k is scaled by state^(-1/2); each head's
+      output is RMS-normed without a weight and multiplied by a SiLU gate.
+    * kind "wkv": a decay per state ROW and token, S_t = diag(a_t) S_(t-1) +
+      k_t v_t^T with a_t = exp(-exp(z_t)), z_t a rank-`decay_rank` function
+      of the token; a token reads y_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t;
+      q, k, v, the gate and z are read from five blends of the token's row
+      with the previous token's (kept in the state slot); each head's output
+      is RMS-normed, weighted and multiplied by a SiLU gate.
+    * kind "mlstm": log gates i (tanh-capped at `gate_cap`) and f =
+      logsigmoid(capped) per head and token, a running maximum m_t = max(f +
+      m_(t-1), i) from 0, a_t = exp(f + m_(t-1) - m_t), b_t = exp(i - m_t);
+      a normaliser n runs along with v = 1 and y_t = S_t^T q_t / (max(|n_t .
+      q_t|, exp(-m_t)) + 1e-6), q scaled by state^(-1/2); each head's output
+      is RMS-normed, weighted and multiplied by a sigmoid gate."""
     kind: str
     heads: int
     state: int                          # rows of the state = size of k and q
@@ -212,6 +227,15 @@ class ScanMixerSpec:
     conv: int = 0                       # taps of the causal convolution
     norm_groups: int = 1
     decay: tuple | None = None
+    rot: RotarySpec = RotarySpec()
+    gate_cap: float = 0.0
+    decay_rank: int = 0
+
+    @property
+    def extra_state(self) -> int:
+        """fp32 values per head kept beside the matrix state: the
+        normaliser and the running maximum."""
+        return self.state + 1 if self.kind == "mlstm" else 0
 
     @property
     def inner(self) -> int:
@@ -236,10 +260,12 @@ class GruMixerSpec:
 class ParallelMixerSpec:
     """Two mixers side by side on the same input (models/parallel_mixer.py):
     softmax attention over the paged pool and a recurrent matrix-state
-    mixer; each output is RMS-normed over the model width with its own
-    weight and the two are averaged."""
+    mixer. Without `scales`, each output is RMS-normed over the model width
+    with its own weight and the two are averaged; with them the result is
+    scales[0] * left + scales[1] * right."""
     left: PagedMixerSpec
     right: ScanMixerSpec
+    scales: tuple | None = None
 
 
 @dataclass(frozen=True)
@@ -270,6 +296,8 @@ class FeedForwardSpec:
     route_correction: bool = False
     group_top: int = 1
     renorm: bool = False
+    # a learned bias per expert on the router's logits (choice AND weights)
+    route_bias: bool = False
 
 
 @dataclass(frozen=True)
@@ -280,6 +308,9 @@ class LayerSpec:
     mixer: ("LatentMixerSpec | PagedMixerSpec | ScanMixerSpec"
             " | ParallelMixerSpec | GruMixerSpec")
     mlp: FeedForwardSpec | None = None
+    # >= 0: the layer runs with the weights of that layer (and a cache and
+    # state of its own); the rest of the entry is the same
+    weights_of: int = -1
 
 
 @dataclass
@@ -485,9 +516,30 @@ class ModelSpec:
             return 0
         n = sum(sh[0] * sh[1] * sh[2] * 4 + sh[3] * sh[4] * dtype_size
                 for sh in self.state_pool_shapes() if sh is not None)
-        if self.token_shift:
-            n += len(self.layer_runs()) * self.hidden_size * dtype_size
+        n += 4 * sum(sh[0] * sh[1] for sh in self.extra_state_shapes()
+                     if sh is not None)
+        n += sum(self.shifted_runs()) * self.hidden_size * dtype_size
         return n
+
+    def extra_state_shapes(self) -> list[tuple | None]:
+        """Per layer run: None, or (heads, fp32 values per head) kept beside
+        the matrix state (ScanMixerSpec.extra_state)."""
+        out = []
+        for i, _ in self.layer_runs():
+            m = self.layers[i].mixer
+            if isinstance(m, ParallelMixerSpec):
+                m = m.right
+            n = m.extra_state if isinstance(m, ScanMixerSpec) else 0
+            out.append((m.heads, n) if n else None)
+        return out
+
+    def shifted_runs(self) -> list[bool]:
+        """Per layer run: whether its mixer reads the previous token's
+        normed row, which the sequence's state slot then carries."""
+        return [self.token_shift
+                or (isinstance(self.layers[i].mixer, ScanMixerSpec)
+                    and self.layers[i].mixer.kind == "wkv")
+                for i, _ in self.layer_runs()]
 
     @property
     def has_state(self) -> bool:
@@ -516,6 +568,8 @@ class ModelSpec:
                 n += (self.bigram_buckets + 1) * h
             for ls in self.layers:
                 m = ls.mixer
+                if ls.weights_of >= 0:
+                    continue
                 if self.streams:
                     n += self._stream_layer_weights(h, ls)
                     continue
@@ -621,14 +675,37 @@ class ModelSpec:
         m, f, s = ls.mixer, ls.mlp, self.streams
         sub = s * s + 2 * s + h + (h * h + h if self.residual_gate else 0)
         n = sub + (h if self.token_shift else 0)
-        if isinstance(m, GruMixerSpec):
+        if isinstance(m, ParallelMixerSpec):
+            a = m.left
+            qkv = a.qk_dim * (a.heads + a.kv_heads) + a.kv_heads * a.v_dim
+            n += ((h + 1) * qkv + a.heads * a.v_dim * h
+                  + self._scan_weights(h, m.right))
+        elif isinstance(m, ScanMixerSpec):
+            n += self._scan_weights(h, m)
+        elif isinstance(m, GruMixerSpec):
             n += 4 * h * m.width + 2 * m.width
         else:
             qkv = (m.qk_dim * (m.heads + m.kv_heads) + m.kv_heads * m.v_dim)
             n += (h * qkv + qkv * m.conv + m.heads * m.v_dim * h
                   + (m.heads * h if m.out_gate else 0))
-        if f is not None:
-            n += sub + (3 if f.gated else 2) * h * f.ff
+        if f is None:
+            return n
+        n += sub
+        if f.kind == "moe":
+            n += f.experts * ((3 if f.gated else 2) * h * f.ff + h + 1)
+            n += 3 * h * f.shared_ff + (h if f.shared_gated else 0)
+        else:
+            n += (3 if f.gated else 2) * h * f.ff
+        return n
+
+    @staticmethod
+    def _scan_weights(h: int, m) -> int:
+        """Weight count of a retention, wkv or mlstm mixer."""
+        n = h * (2 * m.heads * m.state + 3 * m.inner)      # q, k, v, gate, o
+        if m.kind == "wkv":
+            n += (5 * h + (h + m.inner) * m.decay_rank + 3 * m.inner)
+        elif m.kind == "mlstm":
+            n += 2 * m.heads * (h + 1) + m.inner
         return n
 
     @staticmethod
@@ -1054,7 +1131,124 @@ class ModelSpec:
         )
 
     @classmethod
-    def from_hf_config(cls, cfg: dict) -> "ModelSpec":
+    def _from_sapatar_config(cls, cfg: dict, shapes: dict) -> "ModelSpec":
+        """Sapatar checkpoints list their layers one by one; an entry names
+        its mixer — "retention" (rotated linear attention with constant
+        decays), "wkv" (matrix state with a decay per channel and token,
+        inputs shifted towards the previous token's) or "parallel"
+        (windowed softmax attention and a gated matrix memory side by side)
+        — and a routed expert bank or none, or the layer whose weights it
+        shares. The residual is `streams` parallel fp32 streams. The rank
+        of the wkv decay is the one size only the tensors tell (`shapes`)."""
+        def rotary(r, dim):
+            r = r or {}
+            rot = RotarySpec(dims=int(r.get("dims", 0) or 0),
+                             base=float(r.get("base", 10000.0)),
+                             layout="half")
+            if rot.dims % 2 or rot.dims > dim:
+                raise ValueError("rotary dims must be even and fit the head")
+            return rot
+
+        entries = cfg["layers"]
+
+        def owner(i):
+            seen = set()
+            while entries[i].get("weights_of") is not None:
+                seen.add(i)
+                j = int(entries[i]["weights_of"])
+                if not 0 <= j < len(entries) or j in seen:
+                    raise ValueError("weights_of names no layer with weights")
+                rest = [{k: v for k, v in entries[x].items()
+                         if k != "weights_of"} for x in (i, j)]
+                if rest[0] != rest[1]:
+                    raise ValueError("layers that share weights must agree")
+                i = j
+            return i
+
+        layers = []
+        for i, ent in enumerate(entries):
+            m, kind, own = ent["mixer"], ent["type"], owner(i)
+            if kind == "retention":
+                mixer, mtype = ScanMixerSpec(
+                    kind="retention", heads=int(m["heads"]),
+                    state=int(m["dim"]), vdim=int(m["vdim"]),
+                    groups=int(m["heads"]),
+                    rot=rotary(m.get("rot"), int(m["dim"])),
+                    decay=tuple(float(d) for d in m["decay"])), "scan"
+                if len(mixer.decay) != mixer.heads:
+                    raise ValueError("one decay per head")
+            elif kind == "wkv":
+                rank = shapes.get(f"l{own}.mix.w1", (64,))[0]
+                mixer, mtype = ScanMixerSpec(
+                    kind="wkv", heads=int(m["heads"]), state=int(m["dim"]),
+                    vdim=int(m["dim"]), groups=int(m["heads"]),
+                    decay_rank=int(rank)), "scan"
+            elif kind == "parallel":
+                a, b = m["left"], m["right"]
+                left = PagedMixerSpec(
+                    heads=int(a["heads"]), kv_heads=int(a["kv_heads"]),
+                    qk_dim=int(a["dim"]), v_dim=int(a["vdim"]),
+                    scale=float(a["scale"]), bias=True,
+                    rot=rotary(a.get("rot"), int(a["dim"])),
+                    window=int(a["mask"]["size"]))
+                if left.heads % left.kv_heads:
+                    raise ValueError("heads must be a multiple of kv_heads")
+                if left.window < 1:
+                    raise ValueError("the window must hold a token")
+                right = ScanMixerSpec(
+                    kind="mlstm", heads=int(b["heads"]), state=int(b["dim"]),
+                    vdim=int(b["vdim"]), groups=int(b["heads"]),
+                    gate_cap=float(b["gate_cap"]))
+                if not right.gate_cap > 0:
+                    raise ValueError("gate_cap must be positive")
+                mixer, mtype = ParallelMixerSpec(
+                    left=left, right=right,
+                    scales=(float(m["left_scale"]),
+                            float(m["right_scale"]))), "parallel"
+            else:
+                raise NotImplementedError(
+                    f"Sapatar mixer type {kind!r} is not implemented")
+            f = ent.get("mlp")
+            if not f:
+                ff = None
+            elif f["kind"] == "moe":
+                r = f["router"]
+                ff = FeedForwardSpec(
+                    kind="moe", ff=int(f["expert"]["ff"]), act="silu",
+                    gated=True, experts=int(r["experts"]), top=int(r["top"]),
+                    shared_ff=int(f["shared"]["ff"]), shared_gated=True,
+                    renorm=True, route_bias=True)
+                if not 1 <= ff.top <= ff.experts:
+                    raise ValueError("router sizes do not fit")
+            else:
+                raise NotImplementedError(
+                    f"Sapatar feed-forward kind {f['kind']!r}")
+            layers.append(LayerSpec(mtype, mixer, ff,
+                                    -1 if own == i else own))
+        streams = int(cfg["streams"])
+        if streams < 1:
+            raise ValueError("at least one residual stream")
+        return cls(
+            architecture="Sapatar",
+            vocab_size=int(cfg["vocab"]),
+            hidden_size=int(cfg["width"]),
+            num_layers=len(layers),
+            layers=tuple(layers),
+            num_heads=1, num_kv_heads=1, head_dim=8, intermediate_size=0,
+            rms_norm_eps=float(cfg["norm"]["eps"]),
+            max_position_embeddings=int(
+                cfg.get("max_position_embeddings", 1 << 20)),
+            eos_token_id=int(cfg.get("eos_token_id", -1)),
+            fp32_residual=True, streams=streams,
+        )
+
+    @classmethod
+    def from_hf_config(cls, cfg: dict, shapes: dict | None = None
+                       ) -> "ModelSpec":
+        """`shapes`: tensor name -> shape of the checkpoint beside the
+        config, for the sizes that no config entry names."""
+        if cfg.get("architecture") == "Sapatar" and "architectures" not in cfg:
+            return cls._from_sapatar_config(cfg, shapes or {})
         if cfg.get("architecture") == "Fuvuvik" and "architectures" not in cfg:
             return cls._from_fuvuvik_config(cfg)
         if cfg.get("architecture") == "Makezen" and "architectures" not in cfg:
@@ -1233,7 +1427,24 @@ class ModelSpec:
     @classmethod
     def from_dir(cls, model_dir: str | Path) -> "ModelSpec":
         with open(Path(model_dir) / "config.json") as f:
-            return cls.from_hf_config(json.load(f))
+            cfg = json.load(f)
+        return cls.from_hf_config(cfg, checkpoint_shapes(model_dir)
+                                  if "architectures" not in cfg else None)
+
+
+def checkpoint_shapes(model_dir: str | Path) -> dict[str, tuple]:
+    """Tensor name -> shape, from the headers of a folder's safetensors
+    files (8 bytes of little-endian length, then JSON)."""
+    out: dict[str, tuple] = {}
+    for path in sorted(Path(model_dir).glob("*.safetensors")):
+        with open(path, "rb") as f:
+            n = int.from_bytes(f.read(8), "little")
+            if not 0 < n <= path.stat().st_size - 8:
+                raise ValueError(f"{path}: not a safetensors file")
+            head = json.loads(f.read(n))
+        out.update({k: tuple(v["shape"]) for k, v in head.items()
+                    if k != "__metadata__"})
+    return out
 
 
 # Named presets so the bench / tests / control plane can run with

@@ -250,13 +250,15 @@ class KVCache:
         # recurrent mixers: per layer run a matrix state [slots + 1, heads,
         # state, vdim] in fp32 whatever the engine dtype, and the last
         # inputs of the short convolution [slots + 1, taps - 1, channels]
-        # in the engine dtype; with a token shift also the previous token's
-        # normed row [slots + 1, width] of every run. One slot per live
+        # in the engine dtype; for mixers that shift their input also the
+        # previous token's normed row [slots + 1, width], and for those with
+        # a normaliser its fp32 values [slots + 1, heads, n]. One slot per live
         # sequence (max_num_seqs of them); the extra last slot takes the padded rows of a captured
         # decode graph, as pad_block does for the paged pools
         self.ssm_states: list = [None] * self.num_layers
         self.conv_states: list = [None] * self.num_layers
         self.shift_states: list = [None] * self.num_layers
+        self.extra_states: list = [None] * self.num_layers
         self.state_allocator = None
         self.pad_state_slot = -1
         if self.layered and spec.has_state:
@@ -284,11 +286,15 @@ class KVCache:
                     self.conv_states[r] = torch.zeros(
                         (nslots + 1, crows, cch), dtype=act_dtype,
                         device=device)
-            if spec.token_shift:
-                self.shift_states = [
-                    torch.zeros((nslots + 1, spec.hidden_size),
-                                dtype=act_dtype, device=device)
-                    for _ in range(self.num_layers)]
+            for r, sh in enumerate(spec.extra_state_shapes()):
+                if sh is not None:
+                    self.extra_states[r] = torch.zeros(
+                        (nslots + 1, *sh), dtype=torch.float32, device=device)
+            for r, shifted in enumerate(spec.shifted_runs()):
+                if shifted:
+                    self.shift_states[r] = torch.zeros(
+                        (nslots + 1, spec.hidden_size), dtype=act_dtype,
+                        device=device)
         # last block reserved as the graph-padding scratch block (see
         # engine/graph_runner.py): padded rows write/read there, never live KV
         self.pad_block = num_blocks - 1

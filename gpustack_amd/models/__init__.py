@@ -7,6 +7,7 @@ _MODEL_CLASSES = {
     "Fusipel": ("fusipel", "FusipelForCausalLM"),
     "Livasun": ("livasun", "LivasunForCausalLM"),
     "Makezen": ("makezen", "MakezenForCausalLM"),
+    "Sapatar": ("sapatar", "SapatarForCausalLM"),
     "Fuvuvik": ("fuvuvik", "FuvuvikForCausalLM"),
 }
 

@@ -12,8 +12,9 @@ score * route_scale without renormalising. An optional shared expert runs
 for every token and is scaled by a per-token sigmoid gate. Variants, all
 parameters of FeedForwardSpec (ops.route_topk): sigmoid scores, a learned
 per-expert correction that counts for the choice only, groups ranked by the
-sum of their best few choice scores, chosen weights divided by their sum,
-an ungated shared expert.
+sum of their best few choice scores, chosen weights divided by their sum (of
+softmax scores: a softmax over the chosen logits), an ungated shared expert,
+a bias on the router's logits, experts of the gated form.
 
 Router logits, scores, the gate and the weighted sum are fp32; the router
 and gate rows are fused into one fp32 GEMM on the fp32 stream.
@@ -66,13 +67,16 @@ class DenseFF(nn.Module):
 
 
 class RoutedFF(nn.Module):
-    def __init__(self, width: int, f: FeedForwardSpec, dtype, comm=None):
+    """`out_dtype`: of the block's output (default fp32)."""
+
+    def __init__(self, width: int, f: FeedForwardSpec, dtype, comm=None,
+                 out_dtype=torch.float32):
         super().__init__()
         if comm is not None and comm.tp_size > 1:
             raise NotImplementedError("ungated expert bank is not TP-sharded yet")
         if f.experts % max(f.groups, 1):
             raise ValueError("experts must divide evenly into groups")
-        self.f = f
+        self.f, self.out_dtype = f, out_dtype
         self.e, self.top = f.experts, f.top
         mk = lambda *shape, dt=dtype: nn.Parameter(
             torch.empty(*shape, dtype=dt), requires_grad=False)
@@ -80,6 +84,10 @@ class RoutedFF(nn.Module):
         # rows [0, E): router; row E (when gated): the shared expert's gate
         self.router_w = mk(self.e + (1 if self.gated else 0), width,
                            dt=torch.float32)
+        self.router_b = None
+        if f.route_bias:
+            self.router_b = mk(self.router_w.shape[0], dt=torch.float32)
+            self.router_b.zero_()
         self.correction = (mk(self.e, dt=torch.float32)
                            if f.route_correction else None)
         # the plain softmax / best-member routing keeps its own kernel
@@ -87,10 +95,12 @@ class RoutedFF(nn.Module):
                        or f.group_top != 1 or f.renorm)
         if f.route_scores not in ("softmax", "sigmoid"):
             raise ValueError(f"route_scores {f.route_scores!r}")
-        self.up_w = mk(self.e, f.ff, width)
+        # gated: an expert's rows are gate | up
+        self.parts = 2 if f.gated else 1
+        self.up_w = mk(self.e, self.parts * f.ff, width)
         self.down_w = mk(self.e, width, f.ff)
         if f.shared_ff:
-            self.shared_up_w = mk(f.shared_ff, width)
+            self.shared_up_w = mk(self.parts * f.shared_ff, width)
             self.shared_down_w = mk(width, f.shared_ff)
         else:
             self.shared_up_w = self.shared_down_w = None
@@ -100,6 +110,26 @@ class RoutedFF(nn.Module):
 
         return (ops.grouped_ff_available(h, h.shape[1], self.f.ff)
                 and os.environ.get("GPUSTACK_AMD_FUSED_MOE", "1") == "1")
+
+    def graph_ok(self) -> bool:
+        """A decode step can be captured: the grouped expert kernels run and
+        nothing waits for the host."""
+        import os
+
+        return (self.up_w.dtype == torch.bfloat16
+                and self.up_w.shape[2] % 64 == 0 and self.f.ff % 64 == 0
+                and os.environ.get("GPUSTACK_AMD_FUSED_MOE", "1") == "1")
+
+    def _act(self, u):
+        """The activation behind the up projection (in place), or the gated
+        product of its two halves."""
+        if not self.f.gated:
+            ops.act_inplace(u, self.f.act)
+            return u
+        g = torch.empty(u.shape[0], u.shape[1] // 2, dtype=u.dtype,
+                        device=u.device)
+        ops.act_and_mul(g, u, self.f.act)
+        return g
 
     def _consts(self, TK: int, dev):
         """Per-size constant tensors, kept for the module's lifetime: a
@@ -118,7 +148,7 @@ class RoutedFF(nn.Module):
         dev = h.device
         # x32 None: the router reads h itself (fp32 product of its values)
         logits = F.linear(x32 if x32 is not None else h.float(),
-                          self.router_w)                    # fp32 [T, E(+1)]
+                          self.router_w, self.router_b)     # fp32 [T, E(+1)]
         experts = torch.empty(T, self.top, dtype=torch.int32, device=dev)
         weights = torch.empty(T, self.top, dtype=torch.float32, device=dev)
         if self.scored:
@@ -136,7 +166,6 @@ class RoutedFF(nn.Module):
         TK = T * self.top
         flat = experts.reshape(-1).long()
         order = torch.argsort(flat, stable=True)
-        u = torch.empty(TK, self.f.ff, dtype=h.dtype, device=dev)
         y = torch.empty(TK, W, dtype=h.dtype, device=dev)
         capturing = h.is_cuda and torch.cuda.is_current_stream_capturing()
         if self.fused_ok(h) and (TK <= 32 * self.e or capturing):
@@ -146,6 +175,7 @@ class RoutedFF(nn.Module):
             counts.scatter_add_(0, flat, ones)
             offs = (counts.cumsum(0, dtype=torch.int32) - counts).to(torch.int32)
             s_tok = (order // self.top).to(torch.int32)
+            u = torch.empty(TK, self.f.ff, dtype=h.dtype, device=dev)
             ops.grouped_up_act(u, h, self.up_w, s_tok, offs, counts, self.f.act)
             ops.grouped_down(y, u, self.down_w, offs, counts)
         else:
@@ -153,13 +183,15 @@ class RoutedFF(nn.Module):
             # library GEMMs on contiguous row ranges; one host sync
             counts = torch.bincount(flat, minlength=self.e).tolist()
             xs = h.index_select(0, order // self.top)       # [T*top, W]
+            u = torch.empty(TK, self.parts * self.f.ff, dtype=h.dtype,
+                            device=dev)
             off = 0
             for e, n in enumerate(counts):
                 if n:
                     torch.mm(xs[off:off + n], self.up_w[e].t(),
                              out=u[off:off + n])
                 off += n
-            ops.act_inplace(u, self.f.act)
+            u = self._act(u)
             off = 0
             for e, n in enumerate(counts):
                 if n:
@@ -171,10 +203,9 @@ class RoutedFF(nn.Module):
         inv[order] = ar
         shared = None
         if self.shared_up_w is not None:
-            su = F.linear(h, self.shared_up_w)
-            ops.act_inplace(su, self.f.act)
+            su = self._act(F.linear(h, self.shared_up_w))
             shared = F.linear(su, self.shared_down_w)
-        out = torch.empty(T, W, dtype=torch.float32, device=dev)
+        out = torch.empty(T, W, dtype=self.out_dtype, device=dev)
         ops.moe_combine(out, y, inv.view(T, self.top), weights, shared,
                         logits if self.gated else None, self.e)
         return out

@@ -1,5 +1,6 @@
 """Parallel residual streams (hyper-connections) and the pieces that sit
-between them and a sublayer, for models on the fp32 stream.
+between them and a sublayer, for models on the fp32 stream. The gate and the
+shift are options of a model.
 
 The residual is S streams x_1 .. x_S instead of one. A sublayer f reads a
 learned combination of them and its result goes back to all of them while
@@ -10,7 +11,7 @@ the streams mix, everything from the old streams at once:
 * gate: y is multiplied element by element by sigmoid(W h + b), h = norm(u);
 * token shift: the mixer reads h + (h' - h) * mu instead of h, h' the same
   row of the sequence's previous token, kept in its state slot between
-  steps (engine/kv_cache.py shift_states).
+  steps (engine/kv_cache.py shift_states); several mu give several such rows.
 
 ops.stream_step closes one sublayer and opens the next in one row kernel
 (gate, stream update, combination, RMS norm into the GEMM dtype; in a decode
@@ -26,18 +27,18 @@ from .. import ops
 
 class StreamPort(nn.Module):
     """What connects one sublayer to the streams: the weights a (read), M
-    (mix, [from, to]) and b (write), the RMS norm on the way in and the
-    gate's bias on the way out; the gate's projection belongs to whoever
-    runs its GEMM."""
+    (mix, [from, to]) and b (write), the RMS norm on the way in and, with
+    `gate`, the gate's bias on the way out; the gate's projection belongs to
+    whoever runs its GEMM."""
 
-    def __init__(self, width: int, streams: int):
+    def __init__(self, width: int, streams: int, gate: bool = True):
         super().__init__()
         f32 = lambda *shape: nn.Parameter(
             torch.empty(*shape, dtype=torch.float32), requires_grad=False)
         self.read, self.write = f32(streams), f32(streams)
         self.mix = f32(streams, streams)
         self.norm = f32(width)
-        self.gate_b = f32(width)
+        self.gate_b = f32(width) if gate else None
 
 
 class Streams:
@@ -50,12 +51,12 @@ class Streams:
         self.eps = eps
         self.x = torch.empty(T, streams, W, dtype=torch.float32, device=dev)
         self.h = torch.empty(T, W, dtype=dtype, device=dev)
-        self.hs = torch.empty_like(self.h)
         self._closing = None                # (port, result, gate logits)
         ops.embed_streams(self.x, tokens, embed, scale)
 
-    def close(self, port: StreamPort, a, gate) -> None:
-        """The open sublayer's result; written by the next open / finish."""
+    def close(self, port: StreamPort, a, gate=None) -> None:
+        """The open sublayer's result (and its gate's logits, if it has
+        one); written by the next open / finish."""
         self._closing = (port, a, gate)
 
     def _step(self, read, norm, h, shift=None) -> None:
@@ -72,16 +73,18 @@ class Streams:
         return self.h
 
     def open_shifted(self, port: StreamPort, mu, state, rg):
-        """(h, h shifted towards the previous token's)."""
+        """(h, h shifted towards the previous token's): [T, W] for mu [W],
+        one plane [M, T, W] per row of mu [M, W]."""
+        hs = torch.empty(*mu.shape[:-1], *self.h.shape, dtype=self.h.dtype,
+                         device=self.h.device)
         if rg.single:
             self._step(port.read, port.norm, self.h,
-                       (self.hs, mu, state, rg.row_seq, rg.state_slots,
-                        rg.pos32))
+                       (hs, mu, state, rg.row_seq, rg.state_slots, rg.pos32))
         else:
             self._step(port.read, port.norm, self.h)
-            ops.token_shift(self.hs, self.h, mu, state, rg.seq_first,
-                            rg.seq_rows, rg.state_slots, rg.row_seq, rg.pos32)
-        return self.h, self.hs
+            ops.token_shift(hs, self.h, mu, state, rg.seq_first, rg.seq_rows,
+                            rg.state_slots, rg.row_seq, rg.pos32)
+        return self.h, hs
 
     def finish(self, rows, ones, norm):
         """The streams' sum, normed, at the chosen rows (None: all)."""

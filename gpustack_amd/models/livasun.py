@@ -92,16 +92,8 @@ class LivasunForCausalLM(nn.Module):
         """A decode step can be captured when nothing in it waits for the
         host: every routed feed-forward must take the grouped expert
         kernels (models/experts.py)."""
-        import os
-
-        for layer in self.layers:
-            m = layer.mlp
-            if isinstance(m, RoutedFF) and not (
-                    self.dtype == torch.bfloat16
-                    and self.spec.hidden_size % 64 == 0 and m.f.ff % 64 == 0
-                    and os.environ.get("GPUSTACK_AMD_FUSED_MOE", "1") == "1"):
-                return False
-        return True
+        return all(layer.mlp.graph_ok() for layer in self.layers
+                   if isinstance(layer.mlp, RoutedFF))
 
     @torch.inference_mode()
     def forward(self, token_ids, meta, kv, return_hidden: bool = False,

@@ -1,5 +1,5 @@
 """Recurrent mixers with one matrix state per head and sequence, for models
-on the fp32 stream (ModelSpec.fp32_residual). Both run the same recurrence
+on the fp32 stream (ModelSpec.fp32_residual). The first two run the recurrence
 
     S_t = a_t S_(t-1) + b_t k_t v_t^T,    y_t = S_t^T q_t (+ skip * v_t)
 
@@ -27,6 +27,13 @@ states. Nothing is kept per token.
   the scan, g_t = exp(-exp(A_log) softplus(a + dt_bias)), beta_t =
   sigmoid(b); each head's output is RMS-normed, weighted and multiplied by
   silu(gate).
+
+* RetentionMixer, WkvMixer and MlstmMixer are matrix memories
+  (ops.memory_scan): rotated q / k and a constant decay per head; a decay
+  per state row and token with a bonus for the current token, its operands
+  read from rows shifted towards the previous token's; exponential input and
+  forget gates with a running maximum and a normaliser, kept beside the
+  state. Each head's output is RMS-normed, (weighted) and gated.
 
 * MinGruMixer keeps one value per channel instead of a matrix
   (ops.gru_scan), S_t = (1 - z_t) S_(t-1) + z_t c_t: one projection gives z
@@ -207,6 +214,120 @@ class MinGruMixer(nn.Module):
         return self.comm.all_reduce(out) if self.comm is not None else out
 
 
+class _MemoryMixer(nn.Module):
+    """What the matrix memories share: the per-head RMS norm with its gate
+    behind the scan, and the output projection."""
+
+    def __init__(self, width: int, m: ScanMixerSpec, eps: float, dtype, comm,
+                 weighted: bool, gate_mode: int):
+        super().__init__()
+        if comm is not None and comm.tp_size > 1:
+            raise NotImplementedError(
+                "recurrent mixers are not sharded for tensor parallelism yet")
+        self.m, self.eps, self.comm = m, eps, comm
+        self.gate_mode = gate_mode              # ops.gated_group_norm
+        self.nqk = m.heads * m.state
+        if weighted:
+            self.norm = _mk(m.inner, dt=torch.float32)
+        else:
+            self.register_buffer("norm", torch.ones(m.inner), persistent=False)
+        self.o_w = _mk(width, m.inner, dt=dtype)
+
+    def _scan(self, q, k, v, meta, state, **kw):
+        rg = meta.ragged
+        y = torch.empty(q.shape[0], self.m.inner, dtype=torch.float32,
+                        device=q.device)
+        ops.memory_scan(y, q, k, v, state, rg.seq_first, rg.seq_rows,
+                        rg.state_slots, rg.pos32, single=rg.single, **kw)
+        return y
+
+    def _norm(self, y, gate):
+        g = torch.empty(y.shape, dtype=gate.dtype, device=y.device)
+        ops.gated_group_norm(g, y, gate, self.norm, self.m.heads, self.eps,
+                             self.gate_mode)
+        return g
+
+    def forward(self, h, *args, **kw):
+        out = F.linear(self.rows(h, *args, **kw), self.o_w)
+        return self.comm.all_reduce(out) if self.comm is not None else out
+
+
+class RetentionMixer(_MemoryMixer):
+    def __init__(self, width, m, eps, dtype, comm=None):
+        super().__init__(width, m, eps, dtype, comm, False, 2)
+        # rows: q | k | v | gate
+        self.in_w = _mk(2 * self.nqk + 2 * m.inner, width, dt=dtype)
+        f64 = torch.float64
+        self.register_buffer("decay", torch.tensor(m.decay, dtype=f64).float(),
+                             persistent=False)
+        self.register_buffer(
+            "inv_freq", torch.tensor(m.rot.inv_freq(), dtype=f64).float(),
+            persistent=False)
+
+    def rows(self, h, meta, state, tables=None):
+        """`tables`: a dict that lives for one model step; layers with the
+        same rotation share its table of angles there."""
+        m, n = self.m, self.nqk
+        rot = None
+        if m.rot.dims and not meta.ragged.single:
+            tables = {} if tables is None else tables
+            if m.rot not in tables:
+                tables[m.rot] = ops.rope_table(meta.ragged.pos32,
+                                               self.inv_freq)
+            rot = tables[m.rot]
+        u = F.linear(h, self.in_w)
+        y = self._scan(u[:, :n], u[:, n:2 * n], u[:, 2 * n:2 * n + m.inner],
+                       meta, state, k_scale=m.state ** -0.5, decay=self.decay,
+                       inv_freq=self.inv_freq, rot=rot)
+        return self._norm(y, u[:, 2 * n + m.inner:])
+
+
+class WkvMixer(_MemoryMixer):
+    def __init__(self, width, m, eps, dtype, comm=None):
+        super().__init__(width, m, eps, dtype, comm, True, 2)
+        if m.vdim != m.state:
+            raise ValueError("wkv heads are square")
+        f32 = torch.float32
+        self.mu = _mk(5, width, dt=f32)         # r, k, v, gate, decay
+        # transposed, [in, out]: the right operand of one batched product
+        self.rkvg_w = _mk(4, width, m.inner, dt=dtype)
+        self.w1 = _mk(m.decay_rank, width, dt=dtype)
+        self.w2 = _mk(m.inner, m.decay_rank, dt=dtype)
+        self.w0 = _mk(m.inner, dt=f32)
+        self.bonus = _mk(m.heads, m.state, dt=f32)
+
+    def rows(self, hs, meta, state):
+        """hs [5, T, width]: the row shifted by each of mu."""
+        r, k, v, g = torch.bmm(hs[:4], self.rkvg_w)
+        z = F.linear(hs[4], self.w1)
+        ops.act_inplace(z, "tanh")
+        y = self._scan(r, k, v, meta, state, chan=F.linear(z, self.w2),
+                       w0=self.w0, bonus=self.bonus)
+        return self._norm(y, g)
+
+
+class MlstmMixer(_MemoryMixer):
+    def __init__(self, width, m, eps, dtype, comm=None):
+        super().__init__(width, m, eps, dtype, comm, True, 0)
+        # rows: q | k | v | gate | i | f, zero rows up to a multiple of 8 so
+        # that every row of the product starts on a 16-byte boundary
+        self.col_g = 2 * self.nqk + m.inner
+        self.col_i = self.col_g + m.inner
+        n = self.col_i + 2 * m.heads
+        self.in_w = _mk((n + 7) // 8 * 8, width, dt=dtype)
+        self.in_w.zero_()
+        self.i_b = _mk(m.heads, dt=torch.float32)
+        self.f_b = _mk(m.heads, dt=torch.float32)
+
+    def rows(self, h, meta, state, extra):
+        m, n, g, i = self.m, self.nqk, self.col_g, self.col_i
+        u = F.linear(h, self.in_w)
+        y = self._scan(u[:, :n], u[:, n:2 * n], u[:, 2 * n:g], meta, state,
+                       q_scale=m.state ** -0.5, gates=u[:, i:i + 2 * m.heads],
+                       i_b=self.i_b, f_b=self.f_b, cap=m.gate_cap, extra=extra)
+        return self._norm(y, u[:, g:i])
+
+
 def build_scan_mixer(width: int, m: ScanMixerSpec, eps: float, dtype,
                      comm=None):
     if m.kind == "delta":
@@ -215,4 +336,8 @@ def build_scan_mixer(width: int, m: ScanMixerSpec, eps: float, dtype,
         return Mamba2Mixer(width, m, eps, dtype, comm)
     if m.kind == "lightning":
         return LightningMixer(width, m, eps, dtype, comm)
+    memory = {"retention": RetentionMixer, "wkv": WkvMixer,
+              "mlstm": MlstmMixer}.get(m.kind)
+    if memory is not None:
+        return memory(width, m, eps, dtype, comm)
     raise NotImplementedError(f"recurrent mixer kind {m.kind!r}")

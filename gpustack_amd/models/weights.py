@@ -66,8 +66,12 @@ def _layered_tensor_plan(model):
         plan.append(("final.norm.b", model.final_norm_b, same))
     if not getattr(model, "tied_head", False):
         plan.append(("head", model.lm_head, same))
+    seen = set()
     for i, layer in enumerate(model.layers):
         p = f"l{i}."
+        if id(layer) in seen:
+            continue                    # runs with an earlier layer's weights
+        seen.add(id(layer))
         if hasattr(layer, "port1"):
             plan += _stream_layer_plan(p, layer)
             continue
@@ -186,18 +190,19 @@ def _delta_mixer_plan(p: str, a):
 
 
 def _head_norm_attention_plan(p: str, a):
-    """Plan entries of a paged attention mixer with biases and per-head
-    q / k norms (models/paged_attention.py)."""
+    """Plan entries of a paged attention mixer with biases and (optional)
+    per-head q / k norms (models/paged_attention.py)."""
     same = lambda t: t
     nq, nk = a.nq, a.nk
-    return [
+    norms = [] if a.q_head_norm is None else [
+        (p + "q.norm", a.q_head_norm, same),
+        (p + "k.norm", a.k_head_norm, same)]
+    return norms + [
         (p + "q", a.qkv_w[:nq], same), (p + "k", a.qkv_w[nq:nq + nk], same),
         (p + "v", a.qkv_w[nq + nk:], same),
         (p + "q.b", a.qkv_b[:nq], same),
         (p + "k.b", a.qkv_b[nq:nq + nk], same),
-        (p + "v.b", a.qkv_b[nq + nk:], same),
-        (p + "q.norm", a.q_head_norm, same),
-        (p + "k.norm", a.k_head_norm, same), (p + "o", a.o_w, same),
+        (p + "v.b", a.qkv_b[nq + nk:], same), (p + "o", a.o_w, same),
     ]
 
 
@@ -251,6 +256,66 @@ def _sandwich_ln_layer_plan(p: str, layer):
     return plan
 
 
+def _stream_port_plan(p: str, layer):
+    """Plan entries of the two sublayers' stream weights, norms and (gated
+    sublayers) gate biases, all fp32."""
+    same = lambda t: t
+    plan = []
+    for q, port in (("1", layer.port1), ("2", layer.port2)):
+        if port is not None:
+            plan += [(p + "norm" + q, port.norm, same),
+                     (p + f"hc{q}.in", port.read, same),
+                     (p + f"hc{q}.out", port.write, same),
+                     (p + f"hc{q}.mix", port.mix, same)]
+            if port.gate_b is not None:
+                plan.append((p + f"rg{q}.b", port.gate_b, same))
+    return plan
+
+
+def _memory_mixer_plan(p: str, a):
+    """Plan entries of a retention, mlstm or wkv mixer
+    (models/state_mixers.py): the projections that read the same row fuse
+    into one; the wkv projections read a row each and are stored transposed,
+    stacked for one batched product."""
+    same = lambda t: t
+    kind, n, i = a.m.kind, a.nqk, a.m.inner
+    plan = [(p + "o", a.o_w, same)]
+    if kind == "wkv":
+        W = a.mu.shape[1]
+        plan += [(p + "mu." + nm, a.mu[j], same) for j, nm in enumerate("rkvgw")]
+        plan += [(p + nm, a.rkvg_w[j], _shaped(lambda t: t.t(), i, W))
+                 for j, nm in enumerate("rkvg")]
+        return plan + [
+            (p + "w1", a.w1, same), (p + "w2", a.w2, same),
+            (p + "w0", a.w0, same), (p + "u", a.bonus, same),
+            (p + "norm", a.norm, same)]
+    plan += [(p + "q", a.in_w[:n], same), (p + "k", a.in_w[n:2 * n], same),
+             (p + "v", a.in_w[2 * n:2 * n + i], same),
+             (p + "g", a.in_w[2 * n + i:2 * n + 2 * i], same)]
+    if kind == "mlstm":
+        c, h = a.col_i, a.m.heads
+        plan += [(p + "i", a.in_w[c:c + h], same),
+                 (p + "f", a.in_w[c + h:c + 2 * h], same),
+                 (p + "i.b", a.i_b, same), (p + "f.b", a.f_b, same),
+                 (p + "norm", a.norm, same)]
+    return plan
+
+
+def _memory_layer_plan(p: str, layer):
+    """Plan entries of one layer on parallel residual streams whose mixer is
+    a matrix memory, alone or beside softmax attention, with a routed expert
+    bank (models/sapatar.py)."""
+    plan = _stream_port_plan(p, layer)
+    if layer.kind == "scan":
+        plan += _memory_mixer_plan(p + "mix.", layer.mixer)
+    else:
+        plan += _head_norm_attention_plan(p + "mix.left.", layer.mixer.left)
+        plan += _memory_mixer_plan(p + "mix.right.", layer.mixer.right)
+    if layer.mlp is not None:
+        plan += _routed_ff_plan(p, layer.mlp)
+    return plan
+
+
 def _stream_layer_plan(p: str, layer):
     """Plan entries of one layer on parallel residual streams with gated
     sublayers and shifted mixer inputs (models/fuvuvik.py): q, k, v and the
@@ -259,14 +324,9 @@ def _stream_layer_plan(p: str, layer):
     another; stream weights, shifts, biases and convolutions stay fp32."""
     same = lambda t: t
     a = layer.mixer
-    plan = []
-    for q, port in (("1", layer.port1), ("2", layer.port2)):
-        if port is not None:
-            plan += [(p + "norm" + q, port.norm, same),
-                     (p + f"hc{q}.in", port.read, same),
-                     (p + f"hc{q}.out", port.write, same),
-                     (p + f"hc{q}.mix", port.mix, same),
-                     (p + f"rg{q}.b", port.gate_b, same)]
+    if layer.kind in ("scan", "parallel"):
+        return _memory_layer_plan(p, layer)
+    plan = _stream_port_plan(p, layer)
     plan += [(p + "shift", layer.shift, same),
              (p + "rg1", layer.gate1_w, same), (p + "mix.o", a.o_w, same)]
     if layer.kind == "gru":
@@ -298,13 +358,22 @@ def _routed_ff_plan(p: str, m):
     """Plan entries of a routed expert bank (models/experts.py)."""
     same = lambda t: t
     plan = [(p + "mlp.router", m.router_w[:m.e], same)]
+    if m.router_b is not None:
+        plan.append((p + "mlp.router.b", m.router_b[:m.e], same))
+
+    def up(name, w, ff):
+        # the gated form keeps its gate rows in front of the up rows
+        if m.f.gated:
+            plan.append((name + "gate", w[:ff], same))
+            w = w[ff:]
+        plan.append((name + "up", w, same))
     if getattr(m, "correction", None) is not None:
         plan.append((p + "mlp.correction", m.correction, same))
     for e in range(m.e):
-        plan.append((p + f"mlp.e{e}.up", m.up_w[e], same))
+        up(p + f"mlp.e{e}.", m.up_w[e], m.f.ff)
         plan.append((p + f"mlp.e{e}.down", m.down_w[e], same))
     if m.shared_up_w is not None:
-        plan.append((p + "mlp.shared.up", m.shared_up_w, same))
+        up(p + "mlp.shared.", m.shared_up_w, m.f.shared_ff)
         plan.append((p + "mlp.shared.down", m.shared_down_w, same))
         if m.gated:
             plan.append((p + "mlp.shared.sg", m.router_w[m.e:], same))
@@ -381,7 +450,10 @@ def _random_init_layered(model, cfg: EngineConfig) -> None:
             continue
         if dst.dim() == 1 and not name.endswith(("router", "sg")):
             leaf = name.rsplit(".", 1)[-1]
-            if leaf in ("b", "sink", "lq1", "lk1", "lq2", "lk2"):
+            if ".mu." in name or leaf == "w0":
+                # shifts inside (0, 1); decays a few tokens to dozens long
+                base, std = (0.5, 0.2) if leaf != "w0" else (-2.0, 1.0)
+            elif leaf in ("b", "sink", "lq1", "lk1", "lq2", "lk2"):
                 base, std = 0.0, 0.3     # biases, sinks, lambda vectors
             elif leaf in ("vmix", "correction", "dt_bias", "A_log", "shift"):
                 # blend weight in (0, 1); small choice corrections; step

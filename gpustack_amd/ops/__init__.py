@@ -413,7 +413,7 @@ def _lat_backend(t: torch.Tensor):
     return _load_latent() if t.is_cuda else None
 
 
-ACT_MODES = {"relu2": 0, "gelu": 1, "gelu_tanh": 2, "silu": 3}
+ACT_MODES = {"relu2": 0, "gelu": 1, "gelu_tanh": 2, "silu": 3, "tanh": 4}
 
 
 def embed_pair_hash(x, h, tokens, prev, embed, pair_table, buckets: int,
@@ -556,6 +556,8 @@ def grouped_ff_available(x, width: int, ff: int) -> bool:
 
 
 def grouped_up_act(u, x, up_w, s_tok, offs, counts, mode: str) -> None:
+    """up_w [E, ff, W], or [E, 2 ff, W] (gate rows, then up rows) for the
+    gated form."""
     _load_latent().grouped_up_act(u, x, up_w, s_tok, offs, counts,
                                   ACT_MODES[mode])
 
@@ -929,6 +931,39 @@ def delta_scan(y, src, col_q: int, col_k: int, col_v: int, gate_src,
                              pos32)
 
 
+def rope_table(pos32, inv_freq):
+    """cos / sin of pos * f for every row, [T, 2, half] fp32: the table a
+    prompt's memory_scan reads (None on the CPU, whose reference turns the
+    rows itself)."""
+    if not pos32.is_cuda:
+        return None
+    out = torch.empty(pos32.numel(), 2, inv_freq.numel(), dtype=torch.float32,
+                      device=pos32.device)
+    _load_state().rope_table(out, pos32, inv_freq)
+    return out
+
+
+def memory_scan(y, q, k, v, state, seq_first, seq_rows, state_slots, pos32, *,
+                q_scale: float = 1.0, k_scale: float = 1.0, decay=None,
+                chan=None, w0=None, bonus=None, gates=None, i_b=None,
+                f_b=None, cap: float = 0.0, extra=None, inv_freq=None,
+                rot=None, single: bool = False) -> None:
+    """Matrix memory over the state pool (torch_ref.memory_scan has the
+    semantics). `single`: every sequence brings one row (a decode step).
+    `rot`: the step's rope_table, shared by the layers of a prompt (None: the
+    op makes its own)."""
+    b = _state_backend(q)
+    if b is not None:
+        b.memory_scan(y, q, k, v, q_scale, k_scale, decay, chan, w0, bonus,
+                      rot, inv_freq, gates, i_b, f_b, cap, state, extra,
+                      seq_first, seq_rows, state_slots, pos32, single)
+    else:
+        torch_ref.memory_scan(y, q, k, v, state, seq_first, seq_rows,
+                              state_slots, pos32, q_scale, k_scale, decay,
+                              chan, w0, bonus, gates, i_b, f_b, cap, extra,
+                              inv_freq)
+
+
 # --- parallel residual streams, token shift, gated recurrence --------------
 # ops/csrc/hyperrows32.hip, gru_scan.hip and short_conv.hip in
 # `_hip_streams.so`.
@@ -974,7 +1009,8 @@ def stream_step(x, a, gate, gate_b, mix, out_w, in_w, norm_w, eps: float, h,
     """Close one sublayer on the streams and open the next
     (torch_ref.stream_step has the semantics). `shift` = (hs, mu, state,
     row_seq, state_slots, pos32), for batches of single rows: the token
-    shift of h runs in the same launch."""
+    shift of h (one or several, as in token_shift) runs in the same
+    launch."""
     k = _streams_backend(x)
     if k is not None:
         k.stream_step(x, a, gate, gate_b, mix, out_w, in_w, norm_w, eps, h,

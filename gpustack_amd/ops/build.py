@@ -38,7 +38,8 @@ PAGED_SOURCES = ["rowmix32.hip", "roperows32.hip", "ragged_attn.hip",
 # stores come with rowmix32.hip)
 STATE_SO_PATH = PKG_DIR / "_hip_state.so"
 STATE_SOURCES = ["lnrows32.hip", "state_scan.hip", "delta_scan.hip",
-                 "short_conv.hip", "rowmix32.hip", "state_bindings.cpp"]
+                 "memory_scan.hip", "short_conv.hip", "rowmix32.hip",
+                 "state_bindings.cpp"]
 
 # rows of parallel residual streams, token shift, gated recurrence, short
 # convolution

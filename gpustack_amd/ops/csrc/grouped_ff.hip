@@ -1,6 +1,7 @@
-// Grouped ungated expert feed-forward for decode-sized batches (gfx950):
+// Grouped expert feed-forward for decode-sized batches (gfx950):
 //
 //   u[j, :] = act(x[tok_j] . Wu[e_j]^T)        grouped_up_act
+//             (gated: act(x . Wg^T) * (x . Wu^T), Wg the bank's first rows)
 //   y[j, :] = u[j] . Wd[e_j]^T                  grouped_down
 //
 // over the expert-sorted assignment list j (tok_j, per-expert offsets and
@@ -61,8 +62,9 @@ DEVICE_INLINE void gf_stage(unsigned short* lds, const unsigned short* src,
   }
 }
 
-// out[j, N] = f(src_rows(j) [K] . w[e, N, K]^T); GATHER: rows via tok
-template <bool GATHER>
+// out[j, N] = f(src_rows(j) [K] . w[e, N, K]^T); GATHER: rows via tok. GLU:
+// w[e, 2 N, K] and out = f(src . w[:N]^T) * (src . w[N:]^T)
+template <bool GATHER, bool GLU>
 __global__ __launch_bounds__(GF_THREADS) void grouped_ff_kernel(
     unsigned short* __restrict__ out, const unsigned short* __restrict__ src,
     const unsigned short* __restrict__ w, const int* __restrict__ s_tok,
@@ -79,10 +81,11 @@ __global__ __launch_bounds__(GF_THREADS) void grouped_ff_kernel(
   const int lc = lane & 15, lg = lane >> 4;
   __shared__ unsigned short Xl[16 * GF_LD];
   const unsigned short* panel =
-      w + ((long)e * N + nt * GF_BN + wave * 16 + lc) * K;
+      w + ((long)e * (GLU ? 2 * N : N) + nt * GF_BN + wave * 16 + lc) * K;
+  const unsigned short* panel2 = panel + (GLU ? (long)N * K : 0);
   for (int m0 = 0; m0 < cnt; m0 += 16) {
     const int nrows = min(16, cnt - m0);
-    f32x4 acc{0.f, 0.f, 0.f, 0.f};
+    f32x4 acc{0.f, 0.f, 0.f, 0.f}, acc2{0.f, 0.f, 0.f, 0.f};
     for (int k0 = 0; k0 < K; k0 += GF_KC) {
       const int kc = min(GF_KC, K - k0);
       __syncthreads();
@@ -95,6 +98,11 @@ __global__ __launch_bounds__(GF_THREADS) void grouped_ff_kernel(
         const u16x8 b =
             *reinterpret_cast<const u16x8*>(panel + k0 + kk + lg * 8);
         acc = gf_mfma(a, b, acc);
+        if constexpr (GLU) {
+          const u16x8 b2 =
+              *reinterpret_cast<const u16x8*>(panel2 + k0 + kk + lg * 8);
+          acc2 = gf_mfma(a, b2, acc2);
+        }
       };
       if (kc == GF_KC) {
 #pragma unroll
@@ -107,7 +115,8 @@ __global__ __launch_bounds__(GF_THREADS) void grouped_ff_kernel(
     for (int r = 0; r < 4; ++r) {
       const int row = lg * 4 + r;
       if (row >= nrows) continue;
-      const float v = act_mode >= 0 ? gf_act(acc[r], act_mode) : acc[r];
+      float v = act_mode >= 0 ? gf_act(acc[r], act_mode) : acc[r];
+      if constexpr (GLU) v *= acc2[r];
       out[(long)(base + m0 + row) * N + nt * GF_BN + wave * 16 + lc] = f2bf(v);
     }
   }
@@ -119,18 +128,23 @@ __global__ __launch_bounds__(GF_THREADS) void grouped_ff_kernel(
 void grouped_up_act_launch(void* u, const void* x, const void* w,
                            const int* s_tok, const int* offs,
                            const int* counts, int E, int K, int N, int TK,
-                           int T, int act_mode, hipStream_t s) {
+                           int T, int act_mode, int glu, hipStream_t s) {
   if (TK == 0) return;
-  grouped_ff_kernel<true><<<E * (N / GF_BN), GF_THREADS, 0, s>>>(
-      (unsigned short*)u, (const unsigned short*)x, (const unsigned short*)w,
-      s_tok, offs, counts, K, N, TK, T, act_mode);
+  if (glu)
+    grouped_ff_kernel<true, true><<<E * (N / GF_BN), GF_THREADS, 0, s>>>(
+        (unsigned short*)u, (const unsigned short*)x, (const unsigned short*)w,
+        s_tok, offs, counts, K, N, TK, T, act_mode);
+  else
+    grouped_ff_kernel<true, false><<<E * (N / GF_BN), GF_THREADS, 0, s>>>(
+        (unsigned short*)u, (const unsigned short*)x, (const unsigned short*)w,
+        s_tok, offs, counts, K, N, TK, T, act_mode);
 }
 
 void grouped_down_launch(void* y, const void* u, const void* w,
                          const int* offs, const int* counts, int E, int K,
                          int N, int TK, hipStream_t s) {
   if (TK == 0) return;
-  grouped_ff_kernel<false><<<E * (N / GF_BN), GF_THREADS, 0, s>>>(
+  grouped_ff_kernel<false, false><<<E * (N / GF_BN), GF_THREADS, 0, s>>>(
       (unsigned short*)y, (const unsigned short*)u, (const unsigned short*)w,
       nullptr, offs, counts, K, N, TK, TK, -1);
 }

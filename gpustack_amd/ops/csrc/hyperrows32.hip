@@ -8,7 +8,8 @@
 //                   reading and writing the streams once; for batches of
 //                   single rows the token shift of h in the same pass
 //   token_shift   : hs = h + (h_prev - h) * mu, h_prev the row before in the
-//                   sequence, kept in a state slot between steps
+//                   sequence, kept in a state slot between steps; for one
+//                   or several mu, each with a plane of hs of its own
 //
 // The streams x [T, S, W] are updated in place; one workgroup handles a row,
 // a lane reads a channel of ALL streams before it writes any. Norms, gates
@@ -74,13 +75,13 @@ struct StepArgs {
   const float* in;         // [S] or null: nothing to open
   const float* norm_w;     // [W]
   void* h;                 // [T, W]
-  const float* mu;         // [W] or null: no token shift
-  void* hs;                // [T, W]
+  const float* mu;         // [M, W] or null: no token shift
+  void* hs;                // [M, T, W]
   void* prev;              // [nslots, W]
   const int* row_seq;
   const int* slots;
   const int* pos32;
-  int nseq, nslots, S, W;
+  int nseq, nslots, M, T, S, W;
   float eps;
 };
 
@@ -172,7 +173,6 @@ __global__ __launch_bounds__(THREADS) void stream_step_vec_kernel(StepArgs p) {
       if (p.mu != nullptr) {
         TA* pp = (TA*)p.prev + slot * W + i;
         float m[4], q[4] = {0.f, 0.f, 0.f, 0.f};
-        Vec4<float>::load(p.mu + i, m);
         if (has) Vec4<TA>::load(pp, q);
         Vec4<TA>::store(pp, o);
         // the row as the GEMM dtype holds it, as in a longer portion
@@ -180,9 +180,13 @@ __global__ __launch_bounds__(THREADS) void stream_step_vec_kernel(StepArgs p) {
 #pragma unroll
           for (int k = 0; k < 4; ++k) o[k] = bf2f(f2bf(o[k]));
         }
+        for (int b = 0; b < p.M; ++b) {
+          float r[4];
+          Vec4<float>::load(p.mu + (long)b * W + i, m);
 #pragma unroll
-        for (int k = 0; k < 4; ++k) o[k] += (q[k] - o[k]) * m[k];
-        Vec4<TA>::store((TA*)p.hs + t * W + i, o);
+          for (int k = 0; k < 4; ++k) r[k] = o[k] + (q[k] - o[k]) * m[k];
+          Vec4<TA>::store((TA*)p.hs + ((long)b * p.T + t) * W + i, r);
+        }
       }
     }
   }
@@ -233,7 +237,9 @@ __global__ __launch_bounds__(256) void stream_step_kernel(StepArgs p) {
       TA* pp = (TA*)p.prev + slot * W + i;
       const float q = has ? ld(pp) : 0.f, v = ld(&o);
       *pp = o;
-      st((TA*)p.hs + t * W + i, v + (q - v) * p.mu[i]);
+      for (int b = 0; b < p.M; ++b)
+        st((TA*)p.hs + ((long)b * p.T + t) * W + i,
+           v + (q - v) * p.mu[(long)b * W + i]);
     }
   }
 }
@@ -245,7 +251,7 @@ struct ShiftArgs {
   const int* slots;
   const int* row_seq;
   const int* pos32;
-  int nseq, nslots, T, W;
+  int nseq, nslots, M, T, W;
 };
 
 // grid (T, ceil(W / (256 * V))): a lane takes V channels of one row. The
@@ -273,16 +279,19 @@ __global__ __launch_bounds__(256) void token_shift_kernel(
     const long last = min(max(t + p.seq_rows[s] - 1, t), (long)p.T - 1);
     *pp = *reinterpret_cast<const vec_t*>(h + last * W + i);
   }
-  vec_t o;
+  for (int b = 0; b < p.M; ++b) {
+    const float* mu = p.mu + (long)b * W + i;
+    vec_t o;
 #pragma unroll
-  for (int k = 0; k < V; ++k) {
-    const TA cv = cur[k], ov = old[k];
-    const float c = ld(&cv), q = ld(&ov);
-    TA r;
-    st(&r, c + (q - c) * p.mu[i + k]);
-    o[k] = r;
+    for (int k = 0; k < V; ++k) {
+      const TA cv = cur[k], ov = old[k];
+      const float c = ld(&cv), q = ld(&ov);
+      TA r;
+      st(&r, c + (q - c) * mu[k]);
+      o[k] = r;
+    }
+    *reinterpret_cast<vec_t*>(hs + ((long)b * p.T + t) * W + i) = o;
   }
-  *reinterpret_cast<vec_t*>(hs + t * W + i) = o;
 }
 
 template <typename TA>
@@ -306,7 +315,8 @@ __global__ __launch_bounds__(256) void token_shift_any_kernel(
     *pp = h[last * W + i];
   }
   const float c = ld(&cur), q = ld(&old);
-  st(hs + t * W + i, c + (q - c) * p.mu[i]);
+  for (int b = 0; b < p.M; ++b)
+    st(hs + ((long)b * p.T + t) * W + i, c + (q - c) * p.mu[(long)b * W + i]);
 }
 
 template <typename TW>
@@ -396,15 +406,15 @@ void stream_step_launch(float* x, const void* a, const void* gate, long ld_gate,
                         const float* in, const float* norm_w, void* h,
                         const float* mu, void* hs, void* prev,
                         const int* row_seq, const int* slots, const int* pos32,
-                        int nseq, int nslots, int T, int S, int W, float eps,
-                        int bf, hipStream_t s) {
+                        int nseq, int nslots, int M, int T, int S, int W,
+                        float eps, int bf, hipStream_t s) {
   if (T <= 0) return;
   StepArgs p;
   p.x = x; p.a = a; p.gate = gate; p.ld_gate = ld_gate; p.gate_b = gate_b;
   p.mix = mix; p.out = out; p.in = in; p.norm_w = norm_w; p.h = h; p.mu = mu;
   p.hs = hs; p.prev = prev; p.row_seq = row_seq; p.slots = slots;
-  p.pos32 = pos32; p.nseq = nseq; p.nslots = nslots; p.S = S; p.W = W;
-  p.eps = eps;
+  p.pos32 = pos32; p.nseq = nseq; p.nslots = nslots; p.M = M; p.T = T;
+  p.S = S; p.W = W; p.eps = eps;
   if (bf) step_run<unsigned short>(p, T, s);
   else step_run<float>(p, T, s);
 }
@@ -412,13 +422,13 @@ void stream_step_launch(float* x, const void* a, const void* gate, long ld_gate,
 void token_shift_launch(void* hs, const void* h, const float* mu, void* prev,
                         const int* seq_first, const int* seq_rows,
                         const int* slots, const int* row_seq, const int* pos32,
-                        int nseq, int nslots, int T, int W, int bf,
+                        int nseq, int nslots, int M, int T, int W, int bf,
                         hipStream_t s) {
   if (T <= 0 || nseq <= 0) return;
   ShiftArgs p;
   p.mu = mu; p.seq_first = seq_first; p.seq_rows = seq_rows; p.slots = slots;
   p.row_seq = row_seq; p.pos32 = pos32; p.nseq = nseq; p.nslots = nslots;
-  p.T = T; p.W = W;
+  p.M = M; p.T = T; p.W = W;
   if (bf) shift_run<unsigned short>(hs, h, prev, p, s);
   else shift_run<float>(hs, h, prev, p, s);
 }

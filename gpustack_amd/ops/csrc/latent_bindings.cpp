@@ -12,11 +12,11 @@ void latent_norm_store_launch(void*, const void*, long, int, const float*, const
 void act_inplace_launch(void*, long, int, int, hipStream_t);
 void softcap_launch(float*, long, float, hipStream_t);
 void route_grouped_topk_launch(int*, float*, const float*, int, int, int, int, int, int, float, hipStream_t);
-void moe_combine_launch(float*, const void*, const int*, const float*, const void*, const float*, int, int, int, int, int, int, hipStream_t);
+void moe_combine_launch(void*, const void*, const int*, const float*, const void*, const float*, int, int, int, int, int, int, int, hipStream_t);
 void argmax_f32_launch(long*, const float*, int, int, hipStream_t);
 void latent_attention_launch(void*, const void*, const void*, const int*, const int*, const int*, int, float, int, int, int, int, int, int, int, int, int, int, int, long, long, long, long, int, float*, float*, hipStream_t);
 int latent_attn_max_rank();
-void grouped_up_act_launch(void*, const void*, const void*, const int*, const int*, const int*, int, int, int, int, int, int, hipStream_t);
+void grouped_up_act_launch(void*, const void*, const void*, const int*, const int*, const int*, int, int, int, int, int, int, int, hipStream_t);
 void grouped_down_launch(void*, const void*, const void*, const int*, const int*, int, int, int, int, hipStream_t);
 int latent_attn_uses_mfma(int, int, int, int);
 
@@ -206,7 +206,7 @@ bool latent_attention_uses_mfma(Tensor cache) {
 
 void act_inplace(Tensor x, long mode) {
   const int bf = act_kind(x, "x");
-  TORCH_CHECK(mode >= 0 && mode <= 3);
+  TORCH_CHECK(mode >= 0 && mode <= 4);
   act_inplace_launch(x.data_ptr(), x.numel(), (int)mode, bf, cur_stream(x));
   HIP_CHECK_LAST();
 }
@@ -240,10 +240,11 @@ void route_grouped_topk(Tensor experts, Tensor weights, Tensor logits,
 
 void moe_combine(Tensor out, Tensor y, Tensor inv, Tensor weights,
                  OptTensor shared, OptTensor gate, long gate_col) {
-  chk(out, "out", at::kFloat);
+  const int out_bf = act_kind(out, "out");
   chk(inv, "inv", at::kInt);
   chk(weights, "weights", at::kFloat);
   const int bf = act_kind(y, "y");
+  TORCH_CHECK(bf || !out_bf, "fp32 expert rows combine into fp32");
   TORCH_CHECK(out.dim() == 2 && y.dim() == 2 && inv.dim() == 2);
   const int T = out.size(0), W = out.size(1), top = inv.size(1);
   TORCH_CHECK(inv.size(0) == T && weights.sizes() == inv.sizes());
@@ -263,13 +264,14 @@ void moe_combine(Tensor out, Tensor y, Tensor inv, Tensor weights,
       ldg = gate->size(1);
     }
   }
-  moe_combine_launch(out.data_ptr<float>(), y.data_ptr(), inv.data_ptr<int>(),
+  moe_combine_launch(out.data_ptr(), y.data_ptr(), inv.data_ptr<int>(),
                      weights.data_ptr<float>(), sp, gp, ldg, (int)gate_col, T,
-                     W, top, bf, cur_stream(out));
+                     W, top, bf, out_bf, cur_stream(out));
   HIP_CHECK_LAST();
 }
 
-// u[TK, F] = act(x[s_tok] . up[e]^T) over the expert-sorted rows
+// u[TK, F] = act(x[s_tok] . up[e]^T) over the expert-sorted rows; a bank of
+// 2 F rows per expert is gate | up: u = act(x . gate^T) * (x . up^T)
 void grouped_up_act(Tensor u, Tensor x, Tensor up, Tensor s_tok, Tensor offs,
                     Tensor counts, long act_mode) {
   chk(u, "u", at::kBFloat16); chk(x, "x", at::kBFloat16);
@@ -279,7 +281,8 @@ void grouped_up_act(Tensor u, Tensor x, Tensor up, Tensor s_tok, Tensor offs,
   TORCH_CHECK(u.dim() == 2 && x.dim() == 2 && up.dim() == 3);
   const int TK = u.size(0), F = u.size(1), T = x.size(0), W = x.size(1);
   const int E = up.size(0);
-  TORCH_CHECK(up.size(1) == F && up.size(2) == W);
+  const bool glu = up.size(1) == 2L * F;
+  TORCH_CHECK((glu || up.size(1) == F) && up.size(2) == W);
   TORCH_CHECK(s_tok.numel() == TK && offs.numel() == E && counts.numel() == E);
   TORCH_CHECK(W % 32 == 0 && F % 64 == 0 && T >= 1,
               "grouped_up_act needs width % 32 == 0 and ff % 64 == 0");
@@ -287,6 +290,7 @@ void grouped_up_act(Tensor u, Tensor x, Tensor up, Tensor s_tok, Tensor offs,
   grouped_up_act_launch(u.data_ptr(), x.data_ptr(), up.data_ptr(),
                         s_tok.data_ptr<int>(), offs.data_ptr<int>(),
                         counts.data_ptr<int>(), E, W, F, TK, T, (int)act_mode,
+                        glu ? 1 : 0,
                         cur_stream(x));
   HIP_CHECK_LAST();
 }

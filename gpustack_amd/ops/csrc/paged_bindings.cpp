@@ -427,7 +427,7 @@ void head_gate(Tensor out, Tensor o_hts, Tensor gate_src, long col) {
 
 void act_inplace(Tensor x, long mode) {
   const int bf = act_kind(x, "x");
-  TORCH_CHECK(mode >= 0 && mode <= 3);
+  TORCH_CHECK(mode >= 0 && mode <= 4);
   act_inplace_launch(x.data_ptr(), x.numel(), (int)mode, bf, cur_stream(x));
   HIP_CHECK_LAST();
 }

@@ -287,6 +287,7 @@ DEVICE_INLINE float act_apply(float z, int mode) {
       const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
       return 0.5f * z * (1.0f + tanhf(u));
     }
+    case 4: return tanhf(z);
     default: return z / (1.0f + expf(-z));                            // silu
   }
 }
@@ -410,9 +411,9 @@ __global__ __launch_bounds__(64) void route_grouped_topk_kernel(
 }
 
 // out[t] = sum_k wt[t,k] * y[inv[t,k]] + sigmoid(gate[t]) * shared[t]
-template <typename TY>
+template <typename TY, typename TO>
 __global__ __launch_bounds__(ROW_THREADS) void moe_combine_kernel(
-    float* __restrict__ out, const TY* __restrict__ y,
+    TO* __restrict__ out, const TY* __restrict__ y,
     const int* __restrict__ inv, const float* __restrict__ wt,
     const TY* __restrict__ shared, const float* __restrict__ gate,
     int ld_gate, int gate_col, int W, int top, int ny) {
@@ -428,7 +429,38 @@ __global__ __launch_bounds__(ROW_THREADS) void moe_combine_kernel(
       acc += wt[t * top + k] *
              ld(y + (long)min(max(inv[t * top + k], 0), ny - 1) * W + i);
     if (shared != nullptr) acc += g * ld(shared + t * W + i);
-    out[t * W + i] = acc;
+    st(out + t * W + i, acc);
+  }
+}
+
+// The same for bf16 rows in and out, W % 8 == 0: 16 bytes per lane.
+__global__ __launch_bounds__(ROW_THREADS) void moe_combine_vec_kernel(
+    unsigned short* __restrict__ out, const unsigned short* __restrict__ y,
+    const int* __restrict__ inv, const float* __restrict__ wt,
+    const unsigned short* __restrict__ shared, const float* __restrict__ gate,
+    int ld_gate, int gate_col, int W, int top, int ny) {
+  const long t = blockIdx.x;
+  float g = 1.f;
+  if (shared != nullptr && gate != nullptr)
+    g = 1.0f / (1.0f + expf(-gate[t * ld_gate + gate_col]));
+  for (int i = threadIdx.x * 8; i < W; i += ROW_THREADS * 8) {
+    float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < top; ++k) {
+      const float w = wt[t * top + k];
+      const u16x8 v = *reinterpret_cast<const u16x8*>(
+          y + (long)min(max(inv[t * top + k], 0), ny - 1) * W + i);
+#pragma unroll
+      for (int x = 0; x < 8; ++x) acc[x] += w * bf2f(v[x]);
+    }
+    if (shared != nullptr) {
+      const u16x8 v = *reinterpret_cast<const u16x8*>(shared + t * W + i);
+#pragma unroll
+      for (int x = 0; x < 8; ++x) acc[x] += g * bf2f(v[x]);
+    }
+    u16x8 o;
+#pragma unroll
+    for (int x = 0; x < 8; ++x) o[x] = f2bf(acc[x]);
+    *reinterpret_cast<u16x8*>(out + t * W + i) = o;
   }
 }
 
@@ -549,6 +581,7 @@ void act_inplace_launch(void* x, long n, int mode, int bf, hipStream_t s) {
       case 0: act_inplace_vec_kernel<0><<<b8, 256, 0, s>>>(xp, n8); break;
       case 1: act_inplace_vec_kernel<1><<<b8, 256, 0, s>>>(xp, n8); break;
       case 2: act_inplace_vec_kernel<2><<<b8, 256, 0, s>>>(xp, n8); break;
+      case 4: act_inplace_vec_kernel<4><<<b8, 256, 0, s>>>(xp, n8); break;
       default: act_inplace_vec_kernel<3><<<b8, 256, 0, s>>>(xp, n8); break;
     }
     return;
@@ -577,19 +610,27 @@ void route_grouped_topk_launch(int* experts, float* weights,
                                                 scale);
 }
 
-void moe_combine_launch(float* out, const void* y, const int* inv,
+void moe_combine_launch(void* out, const void* y, const int* inv,
                         const float* wt, const void* shared, const float* gate,
                         int ld_gate, int gate_col, int T, int W, int top,
-                        int bf, hipStream_t s) {
+                        int bf, int out_bf, hipStream_t s) {
   if (T == 0) return;
-  if (bf)
-    moe_combine_kernel<unsigned short><<<T, ROW_THREADS, 0, s>>>(
-        out, (const unsigned short*)y, inv, wt, (const unsigned short*)shared,
-        gate, ld_gate, gate_col, W, top, T * top);
+  if (bf && out_bf && W % 8 == 0)
+    moe_combine_vec_kernel<<<T, ROW_THREADS, 0, s>>>(
+        (unsigned short*)out, (const unsigned short*)y, inv, wt,
+        (const unsigned short*)shared, gate, ld_gate, gate_col, W, top, T * top);
+  else if (bf && out_bf)
+    moe_combine_kernel<unsigned short, unsigned short><<<T, ROW_THREADS, 0, s>>>(
+        (unsigned short*)out, (const unsigned short*)y, inv, wt,
+        (const unsigned short*)shared, gate, ld_gate, gate_col, W, top, T * top);
+  else if (bf)
+    moe_combine_kernel<unsigned short, float><<<T, ROW_THREADS, 0, s>>>(
+        (float*)out, (const unsigned short*)y, inv, wt,
+        (const unsigned short*)shared, gate, ld_gate, gate_col, W, top, T * top);
   else
-    moe_combine_kernel<float><<<T, ROW_THREADS, 0, s>>>(
-        out, (const float*)y, inv, wt, (const float*)shared, gate, ld_gate,
-        gate_col, W, top, T * top);
+    moe_combine_kernel<float, float><<<T, ROW_THREADS, 0, s>>>(
+        (float*)out, (const float*)y, inv, wt, (const float*)shared, gate,
+        ld_gate, gate_col, W, top, T * top);
 }
 
 void argmax_f32_launch(long* out, const float* logits, int N, int V,

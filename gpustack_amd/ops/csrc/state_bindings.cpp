@@ -1,6 +1,6 @@
 // Torch bindings for the layer-norm row kernels, the head-norm cache write,
 // scored routing (lnrows32.hip), the recurrent mixers (state_scan.hip,
-// delta_scan.hip) and the short convolution (short_conv.hip);
+// delta_scan.hip, memory_scan.hip) and the short convolution (short_conv.hip);
 // page-wise value stores come from rowmix32.hip. Every shape a kernel or its
 // grid assumes is checked here on the host before the launch; VALUES inside
 // index tensors are bounded in the kernels.
@@ -18,6 +18,10 @@ void gated_group_norm_launch(void*, const float*, const void*, long, const float
 int delta_scan_launch(float*, const void*, long, int, int, int, const void*, long, int, int, int, int, int, int, const float*, const float*, float*, const int*, const int*, const int*, const int*, int, int, int, int, int, hipStream_t);
 int delta_scan_max_state();
 int state_scan_max_state();
+int memory_scan_launch(float*, const void*, long, const void*, long, const void*, long, float, float, int, int, int, int, const float*, const void*, long, const float*, const float*, const float*, const float*, int, const void*, long, const float*, const float*, float, float*, float*, float*, float*, const int*, const int*, const int*, const int*, int, int, int, int, int, hipStream_t);
+int memory_scan_max_state();
+int memory_scan_steps(int, int);
+void rope_table_launch(float*, const int*, const float*, int, int, hipStream_t);
 
 #define HIP_CHECK_LAST()                                                     \
   do {                                                                       \
@@ -306,6 +310,121 @@ void delta_scan(Tensor y, Tensor src, long col_q, long col_k, long col_v,
   HIP_CHECK_LAST();
 }
 
+void rope_table(Tensor out, Tensor pos32, Tensor inv_freq) {
+  chk(out, "out", at::kFloat);
+  chk(pos32, "pos32", at::kInt);
+  chk(inv_freq, "inv_freq", at::kFloat);
+  TORCH_CHECK(out.dim() == 3 && out.size(1) == 2 &&
+              out.size(0) == pos32.numel() && out.size(2) == inv_freq.numel(),
+              "the table must be [T, 2, half]");
+  rope_table_launch(out.data_ptr<float>(), pos32.data_ptr<int>(),
+                    inv_freq.data_ptr<float>(), (int)out.size(0),
+                    (int)out.size(2), cur_stream(out));
+  HIP_CHECK_LAST();
+}
+
+// a fp32 vector operand that must be there with n values
+const float* vec(const OptTensor& t, const char* name, long n) {
+  TORCH_CHECK(t.has_value(), name, " is missing");
+  chk(*t, name, at::kFloat);
+  TORCH_CHECK(t->numel() == n, name, " has the wrong size");
+  return t->data_ptr<float>();
+}
+
+void memory_scan(Tensor y, Tensor q, Tensor k, Tensor v, double q_scale,
+                 double k_scale, OptTensor decay, OptTensor chan, OptTensor w0,
+                 OptTensor bonus, OptTensor rot, OptTensor inv_freq,
+                 OptTensor gates, OptTensor i_b, OptTensor f_b, double cap,
+                 Tensor state, OptTensor extra, Tensor seq_first,
+                 Tensor seq_rows, Tensor state_slots, Tensor pos32,
+                 bool single) {
+  chk(y, "y", at::kFloat);
+  chk(state, "state", at::kFloat);
+  const int bf = view_kind(q, "q");
+  TORCH_CHECK(view_kind(k, "k") == bf && view_kind(v, "v") == bf,
+              "q, k and v must share a dtype");
+  TORCH_CHECK(state.dim() == 4 && state.size(0) >= 1,
+              "state must be [slots, heads, state, vdim]");
+  const int H = state.size(1), N = state.size(2), P = state.size(3);
+  const int T = q.size(0);
+  const long HN = (long)H * N;
+  TORCH_CHECK(H >= 1 && N >= 1 && N <= memory_scan_max_state() && P >= 1,
+              "state size unsupported");
+  TORCH_CHECK(q.size(1) == HN && k.size(0) == T && k.size(1) == HN &&
+              v.size(0) == T && v.size(1) == (long)H * P,
+              "operands do not fit the state");
+  TORCH_CHECK(y.dim() == 2 && y.size(0) == T && y.size(1) == (long)H * P);
+  TORCH_CHECK((int)decay.has_value() + (int)chan.has_value() +
+                  (int)gates.has_value() == 1,
+              "one of constant decays, channel decays and gates");
+  const int nseq = seq_view(seq_first, seq_rows, state_slots, pos32, T);
+  int mode = 0, half = 0;
+  long ld_c = 0, ld_g = 0;
+  const void *cp = nullptr, *gp = nullptr;
+  const float *dp = nullptr, *wp = nullptr, *up = nullptr, *rp = nullptr,
+              *fp = nullptr, *ip = nullptr, *bp = nullptr;
+  float *abp = nullptr, *rdp = nullptr, *ep = nullptr;
+  Tensor ws, table;
+  const bool steps = memory_scan_steps(P, single ? 1 : 0);
+  if (decay.has_value()) {
+    dp = vec(decay, "decay", H);
+  } else if (chan.has_value()) {
+    mode = 1;
+    TORCH_CHECK(view_kind(*chan, "chan") == bf && chan->size(0) == T &&
+                chan->size(1) == HN);
+    cp = chan->data_ptr();
+    ld_c = chan->stride(0);
+    wp = vec(w0, "w0", HN);
+    up = vec(bonus, "bonus", HN);
+  } else {
+    mode = 2;
+    TORCH_CHECK(view_kind(*gates, "gates") == bf && gates->size(0) == T &&
+                gates->size(1) == 2 * H && cap > 0);
+    gp = gates->data_ptr();
+    ld_g = gates->stride(0);
+    ip = vec(i_b, "i_b", H);
+    bp = vec(f_b, "f_b", H);
+    TORCH_CHECK(extra.has_value(), "gates need the normaliser's pool");
+    chk(*extra, "extra", at::kFloat);
+    TORCH_CHECK(extra->dim() == 3 && extra->size(0) == state.size(0) &&
+                extra->size(1) == H && extra->size(2) == N + 1);
+    ep = extra->data_ptr<float>();
+    if (!steps) {
+      ws = at::empty({(long)T, (long)H, 3L}, y.options());
+      abp = ws.data_ptr<float>();
+      rdp = abp + (long)T * H * 2;
+    }
+  }
+  if (inv_freq.has_value() && inv_freq->numel() > 0) {
+    TORCH_CHECK(mode == 0, "rotation comes with constant decays");
+    half = inv_freq->numel();
+    fp = vec(inv_freq, "inv_freq", half);
+    TORCH_CHECK(2 * half <= N, "the rotation is wider than a head");
+    if (!steps) {
+      if (rot.has_value()) {
+        table = *rot;
+      } else {
+        table = at::empty({(long)T, 2L, (long)half}, y.options());
+        rope_table(table, pos32, *inv_freq);
+      }
+      chk(table, "rot", at::kFloat);
+      TORCH_CHECK(table.dim() == 3 && table.size(0) == T &&
+                  table.size(1) == 2 && table.size(2) == half);
+      rp = table.data_ptr<float>();
+    }
+  }
+  const int ok = memory_scan_launch(
+      y.data_ptr<float>(), q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0),
+      v.data_ptr(), v.stride(0), (float)q_scale, (float)k_scale, H, N, P, mode,
+      dp, cp, ld_c, wp, up, rp, fp, half, gp, ld_g, ip, bp, (float)cap, abp,
+      rdp, state.data_ptr<float>(), ep, seq_first.data_ptr<int>(),
+      seq_rows.data_ptr<int>(), state_slots.data_ptr<int>(),
+      pos32.data_ptr<int>(), nseq, (int)state.size(0), T, bf, single ? 1 : 0,
+      cur_stream(q));
+  TORCH_CHECK(ok, "state size unsupported");
+  HIP_CHECK_LAST();
+}
+
 void gated_group_norm(Tensor out, Tensor y, Tensor gate, Tensor w, long groups,
                       double eps, long gate_first) {
   chk(y, "y", at::kFloat);
@@ -336,5 +455,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("short_conv", &short_conv);
   m.def("state_scan", &state_scan);
   m.def("delta_scan", &delta_scan);
+  m.def("memory_scan", &memory_scan);
+  m.def("rope_table", &rope_table);
   m.def("gated_group_norm", &gated_group_norm);
 }

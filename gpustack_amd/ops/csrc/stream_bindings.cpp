@@ -8,8 +8,8 @@
 #include <hip/hip_runtime.h>
 
 void embed_streams_launch(float*, const long*, const void*, int, int, int, long, float, int, hipStream_t);
-void stream_step_launch(float*, const void*, const void*, long, const float*, const float*, const float*, const float*, const float*, void*, const float*, void*, void*, const int*, const int*, const int*, int, int, int, int, int, float, int, hipStream_t);
-void token_shift_launch(void*, const void*, const float*, void*, const int*, const int*, const int*, const int*, const int*, int, int, int, int, int, hipStream_t);
+void stream_step_launch(float*, const void*, const void*, long, const float*, const float*, const float*, const float*, const float*, void*, const float*, void*, void*, const int*, const int*, const int*, int, int, int, int, int, int, float, int, hipStream_t);
+void token_shift_launch(void*, const void*, const float*, void*, const int*, const int*, const int*, const int*, const int*, int, int, int, int, int, int, hipStream_t);
 void gru_scan_launch(void*, const void*, long, int, int, int, int, const float*, const float*, float*, const int*, const int*, const int*, const int*, const int*, float*, int, int, int, int, int, hipStream_t);
 int stream_step_max_streams();
 int stream_step_max_width();
@@ -110,7 +110,7 @@ void stream_step(Tensor x, OptTensor a, OptTensor gate, OptTensor gate_b,
               *np = nullptr, *mup = nullptr;
   void *hp = nullptr, *hsp = nullptr, *pp = nullptr;
   const int *rs = nullptr, *sl = nullptr, *ps = nullptr;
-  int nseq = 1, nslots = 1;
+  int nseq = 1, nslots = 1, M = 1;
   if (a.has_value()) {
     kind(act_kind(*a, "a"));
     TORCH_CHECK(a->dim() == 2 && a->size(0) == T && a->size(1) == W);
@@ -137,7 +137,9 @@ void stream_step(Tensor x, OptTensor a, OptTensor gate, OptTensor gate_b,
                   state_slots.has_value() && pos32.has_value());
       kind(act_kind(*hs, "hs"));
       kind(act_kind(*prev, "prev"));
-      TORCH_CHECK(hs->sizes() == h->sizes() && prev->dim() == 2 &&
+      TORCH_CHECK(mu.has_value() && mu->numel() >= W && mu->numel() % W == 0);
+      M = mu->numel() / W;
+      TORCH_CHECK(hs->numel() == (long)M * T * W && prev->dim() == 2 &&
                   prev->size(0) >= 1 && prev->size(1) == W);
       chk(*row_seq, "row_seq", at::kInt);
       chk(*state_slots, "state_slots", at::kInt);
@@ -145,7 +147,7 @@ void stream_step(Tensor x, OptTensor a, OptTensor gate, OptTensor gate_b,
       nseq = state_slots->numel();
       TORCH_CHECK(row_seq->numel() == T && pos32->numel() == T && nseq == T,
                   "the shift in this pass takes one row per sequence");
-      mup = vec(mu, "mu", W);
+      mup = vec(mu, "mu", (long)M * W);
       hsp = hs->data_ptr();
       pp = prev->data_ptr();
       nslots = prev->size(0);
@@ -155,7 +157,7 @@ void stream_step(Tensor x, OptTensor a, OptTensor gate, OptTensor gate_b,
     }
   }
   stream_step_launch(x.data_ptr<float>(), ap, gp, ld_gate, gb, mp, op, ip, np,
-                     hp, mup, hsp, pp, rs, sl, ps, nseq, nslots, T, S, W,
+                     hp, mup, hsp, pp, rs, sl, ps, nseq, nslots, M, T, S, W,
                      (float)eps, bf, cur_stream(x));
   HIP_CHECK_LAST();
 }
@@ -168,17 +170,19 @@ void token_shift(Tensor hs, Tensor h, Tensor mu, Tensor prev, Tensor seq_first,
               "operands must share a dtype");
   chk(mu, "mu", at::kFloat);
   chk(row_seq, "row_seq", at::kInt);
-  TORCH_CHECK(h.dim() == 2 && hs.sizes() == h.sizes() && prev.dim() == 2 &&
-              prev.size(1) == h.size(1) && prev.size(0) >= 1);
+  TORCH_CHECK(h.dim() == 2 && prev.dim() == 2 && prev.size(1) == h.size(1) &&
+              prev.size(0) >= 1);
   TORCH_CHECK(hs.data_ptr() != h.data_ptr(), "hs must not alias h");
   const int T = h.size(0), W = h.size(1);
-  TORCH_CHECK(mu.numel() == W && row_seq.numel() == T);
+  TORCH_CHECK(mu.numel() >= W && mu.numel() % W == 0 && row_seq.numel() == T);
+  const int M = mu.numel() / W;
+  TORCH_CHECK(hs.numel() == (long)M * T * W, "one plane of hs per shift");
   const int nseq = seq_view(seq_first, seq_rows, state_slots, pos32, T);
   token_shift_launch(hs.data_ptr(), h.data_ptr(), mu.data_ptr<float>(),
                      prev.data_ptr(), seq_first.data_ptr<int>(),
                      seq_rows.data_ptr<int>(), state_slots.data_ptr<int>(),
                      row_seq.data_ptr<int>(), pos32.data_ptr<int>(), nseq,
-                     (int)prev.size(0), T, W, bf, cur_stream(h));
+                     (int)prev.size(0), M, T, W, bf, cur_stream(h));
   HIP_CHECK_LAST();
 }
 

@@ -412,6 +412,8 @@ def act_inplace(x: torch.Tensor, mode: str) -> None:
         y = torch.nn.functional.gelu(xf, approximate="tanh")
     elif mode == "silu":
         y = torch.nn.functional.silu(xf)
+    elif mode == "tanh":
+        y = torch.tanh(xf)
     else:
         raise ValueError(mode)
     x.copy_(y.to(x.dtype))
@@ -451,7 +453,7 @@ def moe_combine(out: torch.Tensor, y: torch.Tensor, inv: torch.Tensor,
         if gate_logits is not None:
             sh = sh * torch.sigmoid(gate_logits[:, gate_col:gate_col + 1].float())
         acc = acc + sh
-    out.copy_(acc)
+    out.copy_(acc.to(out.dtype))
 
 
 def softcap_(logits: torch.Tensor, cap: float) -> None:
@@ -956,6 +958,92 @@ def head_gate(out: torch.Tensor, o_hts: torch.Tensor, gate_src: torch.Tensor,
     out.copy_(o.reshape(T, H * VD).to(out.dtype))
 
 
+def memory_scan(y: torch.Tensor, q: torch.Tensor, k: torch.Tensor,
+                v: torch.Tensor, state: torch.Tensor, seq_first: torch.Tensor,
+                seq_rows: torch.Tensor, state_slots: torch.Tensor,
+                pos32: torch.Tensor, q_scale: float = 1.0,
+                k_scale: float = 1.0, decay: torch.Tensor | None = None,
+                chan: torch.Tensor | None = None,
+                w0: torch.Tensor | None = None,
+                bonus: torch.Tensor | None = None,
+                gates: torch.Tensor | None = None,
+                i_b: torch.Tensor | None = None,
+                f_b: torch.Tensor | None = None, cap: float = 0.0,
+                extra: torch.Tensor | None = None,
+                inv_freq: torch.Tensor | None = None) -> None:
+    """Matrix memory, per sequence and head over this step's rows in order,
+    all in fp32; S [N, P] is read from state[slot] (zero when the first row
+    sits at position 0) and written back. q, k [T, H * N] (times q_scale /
+    k_scale; with inv_freq the first 2 * len channels of every head turn by
+    pos * f first, channel i with i + half), v [T, H * P]. One of
+      decay [H]:    S <- decay S + k v^T;  y = S^T q
+      chan [T, H * N] with w0, bonus [H * N]:
+                    y = (S + diag(bonus) k v^T)^T q;
+                    S <- diag(exp(-exp(chan + w0))) S + k v^T
+      gates [T, 2 H] (i | f) with i_b, f_b [H], cap, and the pool extra
+      [slots, H, N + 1] of the normaliser n and the running maximum m:
+                    i = cap tanh((. + i_b) / cap); f = logsigmoid(cap
+                    tanh((. + f_b) / cap)); m' = max(f + m, i);
+                    a = exp(f + m - m'), b = exp(i - m');
+                    S <- a S + b k v^T;  n <- a n + b k;
+                    y = S^T q / (max(|n . q|, exp(-m')) + 1e-6)
+    y: [T, H * P] fp32."""
+    H, N, P = state.shape[1:]
+    T = q.shape[0]
+    qf = q.float().reshape(T, H, N)
+    kf = k.float().reshape(T, H, N)
+    vf = v.float().reshape(T, H, P)
+    half = inv_freq.numel() if inv_freq is not None else 0
+    if half:
+        ang = pos32.to(torch.float32)[:, None] * inv_freq.float()[None, :]
+        c, s = torch.cos(ang)[:, None, :], torch.sin(ang)[:, None, :]
+
+        def turn(t):
+            a, b = t[..., :half], t[..., half:2 * half]
+            return torch.cat([a * c - b * s, b * c + a * s,
+                              t[..., 2 * half:]], -1)
+
+        qf, kf = turn(qf), turn(kf)
+    qf, kf = qf * q_scale, kf * k_scale
+    if chan is not None:
+        w = torch.exp(-torch.exp(chan.float() + w0.float().reshape(-1))
+                      ).reshape(T, H, N)
+        u = bonus.float().reshape(H, N)
+    if gates is not None:
+        g = gates.float()
+        gi = cap * torch.tanh((g[:, :H] + i_b.float()) / cap)
+        z = cap * torch.tanh((g[:, H:] + f_b.float()) / cap)
+        gf = z.clamp(max=0) - torch.log1p(torch.exp(-z.abs()))
+    for sq in range(seq_first.numel()):
+        r0, n, slot = int(seq_first[sq]), int(seq_rows[sq]), int(state_slots[sq])
+        fresh = int(pos32[r0]) <= 0
+        S = torch.zeros_like(state[slot]) if fresh else state[slot].clone()
+        if gates is not None:
+            ex = torch.zeros_like(extra[slot]) if fresh else extra[slot].clone()
+            nv, m = ex[:, :N].clone(), ex[:, N].clone()
+        for t in range(r0, r0 + n):
+            kv = kf[t][:, :, None] * vf[t][:, None, :]
+            if chan is not None:
+                o = ((S + u[:, :, None] * kv) * qf[t][:, :, None]).sum(1)
+                S = w[t][:, :, None] * S + kv
+            elif gates is not None:
+                new = torch.maximum(gf[t] + m, gi[t])
+                a, b = torch.exp(gf[t] + m - new), torch.exp(gi[t] - new)
+                m = new
+                S = a[:, None, None] * S + b[:, None, None] * kv
+                nv = a[:, None] * nv + b[:, None] * kf[t]
+                den = torch.maximum((nv * qf[t]).sum(-1).abs(),
+                                    torch.exp(-m)) + 1e-6
+                o = (S * qf[t][:, :, None]).sum(1) / den[:, None]
+            else:
+                S = decay.float()[:, None, None] * S + kv
+                o = (S * qf[t][:, :, None]).sum(1)
+            y[t] = o.reshape(-1)
+        state[slot] = S
+        if gates is not None:
+            extra[slot] = torch.cat([nv, m[:, None]], -1)
+
+
 # --- parallel residual streams, token shift, gated recurrence --------------
 
 def embed_streams(x: torch.Tensor, tokens: torch.Tensor, embed: torch.Tensor,
@@ -996,14 +1084,17 @@ def token_shift(hs: torch.Tensor, h: torch.Tensor, mu: torch.Tensor,
                 pos32: torch.Tensor) -> None:
     """hs[t] = h[t] + (h_prev - h[t]) * mu with h_prev the row before in the
     same sequence; the row before this step's first one is state[slot] (zero
-    at position 0). The state then holds the step's last row of h."""
+    at position 0). The state then holds the step's last row of h. mu [M, W]
+    with hs [M, T, W]: M shifts of the same rows."""
+    mus = mu.float().reshape(-1, 1, h.shape[1])
+    out = hs.view(mus.shape[0], *h.shape)
     for s in range(seq_first.numel()):
         r0, n, slot = int(seq_first[s]), int(seq_rows[s]), int(state_slots[s])
         x = h[r0:r0 + n].float()
         first = state[slot].float()[None] if int(pos32[r0]) > 0 \
             else torch.zeros_like(x[:1])
         prev = torch.cat([first, x[:-1]], 0)
-        hs[r0:r0 + n] = (x + (prev - x) * mu.float()).to(hs.dtype)
+        out[:, r0:r0 + n] = (x + (prev - x) * mus).to(hs.dtype)
         state[slot] = h[r0 + n - 1].to(state.dtype)
 
 
