@@ -57,13 +57,13 @@ def parse_args():
                          "across ranks, replicated decode); world = tp*cp")
     ap.add_argument("--layer-bench", action="store_true",
                     help="instead of the serving workload: Vunitar, Fusipel, "
-                         "Livasun, Makezen or Fuvuvik layers (--layer-family) at "
+                         "Livasun, Makezen, Fuvuvik or Sapatar layers (--layer-family) at "
                          "real-model sizes beside the closest existing "
                          "stack (prefill/decode tok/s + per-kernel roofline "
                          "shares; gpustack_amd/bench/layer_bench.py)")
     ap.add_argument("--layer-family", default="vunitar",
                     choices=["vunitar", "fusipel", "livasun", "makezen",
-                             "fuvuvik"],
+                             "fuvuvik", "sapatar"],
                     help="model family measured by --layer-bench")
     ap.add_argument("--layer-solo", action="store_true",
                     help="--layer-bench: only the family's own stack end to "

@@ -1,6 +1,7 @@
-"""Layer-level comparison bench: a Vunitar, Fusipel, Livasun, Makezen or
-Fuvuvik stack (`family`) at real-model layer sizes beside the closest llama-lineage stack of equal
-width, depth and heads (random weights, synthetic tokens). Reports end-to-end prefill and decode
+"""Layer-level comparison bench: a Vunitar, Fusipel, Livasun, Makezen, Fuvuvik
+or Sapatar stack (`family`) at real-model layer sizes beside the closest
+existing stacks of equal width, depth and heads (random weights, synthetic
+tokens). Reports end-to-end prefill and decode
 throughput through LLMEngine for both, and per-kernel rates of the new
 kernels next to their counterparts with the fraction of the MI355X
 roofline each reaches (2.5 PFLOP/s dense bf16, 8 TB/s HBM3E).
@@ -190,6 +191,44 @@ def fuvuvik_spec(s, moe: bool = False):
         rms_norm_eps=1e-5, max_position_embeddings=1 << 20, eos_token_id=-1,
         fp32_residual=True, streams=4, token_shift=True, residual_gate=True,
         embed_scale=1.0)
+
+
+def sapatar_spec(s, moe: bool = True):
+    """Layers cycle retention (heads x 128 x 128, all channels rotated),
+    windowed attention (head size 128, heads/4 kv heads, 64 rotated channels,
+    window 1024) beside an mLSTM memory (heads x 128 x 128), wkv (heads of
+    64, decays of rank 64) and retention again, on 4 residual streams; a
+    routed bank of gated SiLU experts, 4 a token, with a shared one."""
+    from ..engine.config import (FeedForwardSpec, LayerSpec, ModelSpec,
+                                 PagedMixerSpec, ParallelMixerSpec,
+                                 RotarySpec, ScanMixerSpec)
+
+    H, W = s["heads"], s["width"]
+    ret = ScanMixerSpec(kind="retention", heads=H, state=128, vdim=128,
+                        groups=H, rot=RotarySpec(dims=128, layout="half"),
+                        decay=tuple(
+                            1.0 - 2.0 ** (-5.0 - 5.0 * h / max(H - 1, 1))
+                            for h in range(H)))
+    left = PagedMixerSpec(heads=H, kv_heads=max(1, H // 4), qk_dim=128,
+                          v_dim=128, scale=128 ** -0.5, bias=True, window=1024,
+                          rot=RotarySpec(dims=64, layout="half"))
+    right = ScanMixerSpec(kind="mlstm", heads=H, state=128, vdim=128, groups=H,
+                          gate_cap=15.0)
+    wkv = ScanMixerSpec(kind="wkv", heads=W // 64, state=64, vdim=64,
+                        groups=W // 64, decay_rank=64)
+    ff = FeedForwardSpec(kind="moe", ff=s["eff"], act="silu", gated=True,
+                         experts=s["experts"], top=4, shared_ff=s["eff"],
+                         shared_gated=True, renorm=True, route_bias=True)
+    cycle = [("scan", ret), ("parallel", ParallelMixerSpec(
+        left=left, right=right, scales=(1.1, 0.7))), ("scan", wkv),
+        ("scan", ret)]
+    return ModelSpec(
+        architecture="Sapatar", vocab_size=32000, hidden_size=W,
+        num_layers=s["layers"],
+        layers=tuple(LayerSpec(*cycle[i % 4], ff) for i in range(s["layers"])),
+        num_heads=1, num_kv_heads=1, head_dim=8, intermediate_size=0,
+        rms_norm_eps=1e-5, max_position_embeddings=1 << 20, eos_token_id=-1,
+        fp32_residual=True, streams=4)
 
 
 def llama_spec(s, moe: bool):
@@ -1146,25 +1185,244 @@ def fuvuvik_kernel_rates(s, device):
     return out
 
 
+def sapatar_kernel_rates(s, device):
+    """Per-kernel rates of the Sapatar kernels next to their likes in the
+    Livasun stack (windowed attention, matrix-state scan and step, its norm,
+    its expert bank) and in the Fuvuvik stack (stream rows, token shift,
+    rotation)."""
+    from .. import ops
+
+    bf = torch.bfloat16
+    H, W, D, BS, S = s["heads"], s["width"], 128, 16, 4
+    G = max(1, H // 4)
+    out = []
+
+    def rec(name, sec, flops=None, nbytes=None, peak=PEAK_FLOPS):
+        if flops is not None:
+            out.append(dict(kernel=name, us=round(sec * 1e6, 1),
+                            tflops=round(flops / sec / 1e12, 1),
+                            roofline=round(flops / sec / peak, 4)))
+        else:
+            out.append(dict(kernel=name, us=round(sec * 1e6, 1),
+                            gbps=round(nbytes / sec / 1e9, 1),
+                            roofline=round(nbytes / sec / PEAK_BW, 4)))
+
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=device)
+    R = lambda *sh: torch.randn(*sh, device=device)
+    slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / H) for h in range(H)],
+                          device=device)
+    # ---- prefill attention: 4 prompts x 2048; decode: 64 x 2048 cached ----
+    win = 1024
+    for phase, nseq, hist, L in (("prefill", 4, 0, 2048), ("decode", 64, 2047, 1)):
+        ctx, T = hist + L, nseq * L
+        nblk = nseq * (ctx // BS) + 1
+        bt = torch.arange(nseq * (ctx // BS), dtype=torch.int32,
+                          device=device).view(nseq, -1)
+        row_seq = torch.arange(nseq, dtype=torch.int32,
+                               device=device).repeat_interleave(L)
+        pos = torch.arange(hist, ctx, dtype=torch.int32, device=device).repeat(nseq)
+        kc, vc = R(nblk, G, BS, D).to(bf), R(nblk, G, D, BS).to(bf)
+        q = R(T, H, D).to(bf)
+        o = torch.empty_like(q)
+        tiles = ops.build_attn_tiles([i * L for i in range(nseq)],
+                                     [hist] * nseq, [L] * nseq, H, G, 1, device)
+        n = nseq * sum(min(i + 1, win) for i in range(hist, ctx))
+        for label, kw in (("window 1024", {}),
+                          ("window 1024 + slopes (Livasun)", dict(slopes=slopes))):
+            sec = _time(lambda: ops.paged_attention(
+                o, q, kc, vc, bt, row_seq, pos, D ** -0.5, tiles=tiles,
+                max_ctx=ctx if L == 1 else 0, window=win, **kw),
+                5 if L > 1 else 20)
+            if L > 1:
+                rec(f"paged_attention {phase}, {label} (mfma, useful pairs)",
+                    sec, flops=4.0 * D * H * n)
+            else:
+                rec(f"paged_attention {phase}, {label} (mfma)", sec,
+                    nbytes=n * G * D * 4)
+
+    # ---- row kernels at T = 8192 rows, and 64 decode rows ----
+    w32, b32 = torch.ones(W, device=device), torch.zeros(W, device=device)
+    mix = torch.eye(S, device=device) * 0.9 + 0.02
+    rw = torch.full((S,), 1.0 / S, device=device)
+    nq, nk = H * D, G * D
+    inv = torch.tensor([10000.0 ** (-i / 32) for i in range(32)], device=device)
+    E, eff, top = s["experts"], s["eff"], 4
+    up, dn = R(E, 2 * eff, W).to(bf), R(E, W, eff).to(bf)
+    for T in (8192, 64):
+        lab = f"{T} rows"
+        x, a = R(T, S, W), R(T, W).to(bf)
+        hb = torch.empty_like(a)
+        h1, h5 = torch.empty_like(a), torch.empty(5, T, W, dtype=bf, device=device)
+        mu1, mu5 = torch.rand(W, device=device), torch.rand(5, W, device=device)
+        state = torch.zeros(65, W, dtype=bf, device=device)
+        nseq = 8 if T > 64 else 64
+        L = T // nseq
+        sf, sr = i32([i * L for i in range(nseq)]), i32([L] * nseq)
+        ss = i32(list(range(nseq)))
+        rs = torch.arange(nseq, dtype=torch.int32, device=device).repeat_interleave(L)
+        p32 = (torch.arange(L, dtype=torch.int32, device=device) + 5).repeat(nseq)
+        step = lambda **kw: _time(lambda: ops.stream_step(
+            x, a, kw.get("gate"), b32 if "gate" in kw else None, mix, rw, rw,
+            w32, 1e-5, hb, shift=kw.get("shift")))
+        rec(f"stream_step (4 streams mixed, norm), {lab}", step(),
+            nbytes=T * W * (8 * S + 4))
+        rec(f"stream_step + gate (Fuvuvik), {lab}", step(gate=R(T, W).to(bf)),
+            nbytes=T * W * (8 * S + 6))
+        if L == 1:
+            rec(f"stream_step + 5 shifts, {lab}",
+                step(shift=(h5, mu5, state, rs, ss, p32)),
+                nbytes=T * W * (8 * S + 18))
+            rec(f"stream_step + 1 shift (Fuvuvik), {lab}",
+                step(shift=(h1, mu1, state, rs, ss, p32)),
+                nbytes=T * W * (8 * S + 10))
+        else:
+            for nm, hh, mu, m in (("5 shifts", h5, mu5, 5),
+                                  ("1 shift (Fuvuvik)", h1, mu1, 1)):
+                rec(f"token_shift, {nm}, {lab}",
+                    _time(lambda: ops.token_shift(hh, hb, mu, state, sf, sr,
+                                                  ss, rs, p32)),
+                    nbytes=T * W * (2 + 2 * m))
+        nblk = T // BS + 1
+        kc = torch.zeros(nblk, G, BS, D, dtype=bf, device=device)
+        vc = torch.zeros(nblk, G, D, BS, dtype=bf, device=device)
+        qkv, qo = R(T, nq + 2 * nk).to(bf), torch.empty(T, nq, dtype=bf, device=device)
+        slots = torch.arange(T, device=device)
+        pg = ops.build_page_groups([0], [0], [T], BS, device) if L > 1 else None
+        for nm, nd in (("rotation + cache write", 0),
+                       ("unit heads + rotation + cache write (Fuvuvik)", D)):
+            rec(f"head_rope_store, {nm}, {lab}",
+                _time(lambda: ops.head_rope_store(
+                    qo, qkv, 0, H, D, None, nd, 0, nq, G, D, None, nd, 0,
+                    nq + nk, inv, True, 1.0, p32, kc, vc, slots, 1e-5,
+                    page_groups=pg)), nbytes=T * (2 * nq + 4 * nk) * 2)
+        y, gt = R(T, nq), R(T, nq).to(bf)
+        wn, go = torch.ones(nq, device=device), torch.empty(T, nq, dtype=bf, device=device)
+        rec(f"gated_group_norm per head, {lab}",
+            _time(lambda: ops.gated_group_norm(go, y, gt, wn, H, 1e-5, 2)),
+            nbytes=T * nq * 8)
+        rec(f"gated_group_norm whole row (Livasun), {lab}",
+            _time(lambda: ops.gated_group_norm(go, y, gt, wn, 1, 1e-5, 0)),
+            nbytes=T * nq * 8)
+        if L > 1:
+            tb = torch.tensor([10000.0 ** (-i / 64) for i in range(64)],
+                              device=device)
+            rec(f"rope_table (once a step), {lab}",
+                _time(lambda: ops.rope_table(p32, tb)), nbytes=T * 64 * 8)
+        # expert bank
+        lg = R(T, E + 1)
+        ex = torch.empty(T, top, dtype=torch.int32, device=device)
+        wt = torch.empty(T, top, device=device)
+        for nm, sig, g in (("softmax", False, 1), ("sigmoid, groups (Livasun)", True, 4)):
+            rec(f"route_topk {nm}, {lab}",
+                _time(lambda: ops.route_topk(ex, wt, lg, None, E, g,
+                                             min(2, g), 2, sig, True, 1.0)),
+                nbytes=T * (E * 4 + top * 8))
+        TK = T * top
+        flat = ex.reshape(-1).long()
+        order = torch.argsort(flat, stable=True)
+        counts = torch.bincount(flat, minlength=E).to(torch.int32)
+        offs = (counts.cumsum(0, dtype=torch.int32) - counts).to(torch.int32)
+        used = int((counts > 0).sum())
+        yx, sh = R(TK, W).to(bf), R(T, W).to(bf)
+        iv = torch.argsort(order).to(torch.int32).view(T, top)
+        for nm, dt, nb in (("bf16 sums", bf, 2), ("fp32 sums (Livasun)", torch.float32, 4)):
+            o = torch.empty(T, W, dtype=dt, device=device)
+            rec(f"moe_combine, {nm}, {lab}",
+                _time(lambda: ops.moe_combine(o, yx, iv, wt, sh, lg, E)),
+                nbytes=T * W * (2 * top + 2 + nb))
+        if L == 1:
+            tok = (order // top).to(torch.int32)
+            u = torch.empty(TK, eff, dtype=bf, device=device)
+            up1 = up[:, :eff].contiguous()
+            rec(f"grouped_up_act gated silu, {lab}",
+                _time(lambda: ops.grouped_up_act(u, hb, up, tok, offs, counts,
+                                                 "silu")),
+                nbytes=used * 2 * eff * W * 2)
+            rec(f"grouped_up_act relu2 (Livasun), {lab}",
+                _time(lambda: ops.grouped_up_act(u, hb, up1, tok, offs, counts,
+                                                 "relu2")),
+                nbytes=used * eff * W * 2)
+            rec(f"grouped_down (both), {lab}",
+                _time(lambda: ops.grouped_down(yx, u, dn, offs, counts)),
+                nbytes=used * eff * W * 2)
+        else:
+            gu, ao = R(TK, 2 * eff).to(bf), torch.empty(TK, eff, dtype=bf, device=device)
+            rec(f"act_and_mul silu, {TK} expert rows",
+                _time(lambda: ops.act_and_mul(ao, gu, "silu")),
+                nbytes=TK * eff * 6)
+            rec(f"act_inplace relu2 (Livasun), {TK} expert rows",
+                _time(lambda: ops.act_inplace(ao, "relu2")), nbytes=TK * eff * 4)
+        del x, yx
+
+    # ---- memories ----
+    inv = torch.tensor([10000.0 ** (-i / 64) for i in range(64)], device=device)
+    for label, nseq, L in (("prefill 8 x 1024", 8, 1024),
+                           ("prefill 1 x 8192", 1, 8192),
+                           ("decode 64 x 1", 64, 1)):
+        T = nseq * L
+        sf, sr = i32([i * L for i in range(nseq)]), i32([L] * nseq)
+        ss = i32(list(range(nseq)))
+        ps = (torch.arange(L, dtype=torch.int32, device=device) + 5).repeat(nseq)
+        dec = torch.full((H,), 0.99, device=device)
+        u = R(T, 4 * nq + 2 * H).to(bf)
+        q, k, v = u[:, :nq], u[:, nq:2 * nq], u[:, 2 * nq:3 * nq]
+        y = torch.empty(T, nq, device=device)
+        st = torch.zeros(nseq + 1, H, D, D, device=device)
+        ext = torch.zeros(nseq + 1, H, D + 1, device=device)
+        b1 = torch.ones(H, device=device)
+        tab = ops.rope_table(ps, inv) if L > 1 else None
+        N6 = W // 64
+        st6 = torch.zeros(nseq + 1, N6, 64, 64, device=device)
+        r6, k6, v6, z6 = R(4, T, W).to(bf)
+        y6 = torch.empty(T, W, device=device)
+        w0, bo = torch.full((W,), -2.0, device=device), torch.ones(N6, 64, device=device)
+        view = (sf, sr, ss, ps)
+        cases = (
+            ("retention", nq * D, lambda: ops.memory_scan(
+                y, q, k, v, st, *view, k_scale=D ** -0.5, decay=dec,
+                inv_freq=inv, rot=tab, single=L == 1)),
+            ("mlstm", nq * D, lambda: ops.memory_scan(
+                y, q, k, v, st, *view, q_scale=D ** -0.5,
+                gates=u[:, 4 * nq:], i_b=b1, f_b=b1, cap=15.0, extra=ext,
+                single=L == 1)),
+            ("wkv", W * 64, lambda: ops.memory_scan(
+                y6, r6, k6, v6, st6, *view, chan=z6, w0=w0, bonus=bo,
+                single=L == 1)),
+            ("state_scan lightning (Livasun)", nq * D, lambda: ops.state_scan(
+                y, u, 2 * nq, nq, 0, None, 0, H, H, D, D, True, None, None,
+                None, dec, st, *view, single=L == 1)))
+        for nm, elems, fn in cases:
+            nm = nm if "state" in nm else f"memory_scan {nm}"
+            sec = _time(fn, 5)
+            if L > 1:
+                rec(f"{nm}, {label} (4 flops per state element)", sec,
+                    flops=4.0 * T * elems, peak=PEAK_VALU)
+            else:
+                rec(f"{nm}, {label} (state read + write)", sec,
+                    nbytes=nseq * elems * 8)
+    return out
+
+
 def run(sizes: list[str], device: str, family: str = "vunitar",
         solo: bool = False) -> None:
     """`solo`: only the family's own stack end to end (no comparison stack,
     no per-kernel rates) — the run to put under a profiler."""
     for name in sizes:
         s = SIZES[name]
-        if family in ("livasun", "makezen", "fuvuvik"):
+        if family in ("livasun", "makezen", "fuvuvik", "sapatar"):
             s = dict(s, layers=4)       # one full cycle of the mixers
         for moe in ((False, True) if family in ("vunitar", "livasun")
-                    else (False,)):
+                    else (family == "sapatar",)):
             row = {"size": name, **s, "ff_kind": "moe" if moe else "dense"}
             mine = {"vunitar": vunitar_spec, "fusipel": fusipel_spec,
                     "livasun": livasun_spec, "makezen": makezen_spec,
-                    "fuvuvik": fuvuvik_spec}[family]
-            # Makezen's and Fuvuvik's closest existing model is another
+                    "fuvuvik": fuvuvik_spec, "sapatar": sapatar_spec}[family]
+            # Makezen's, Fuvuvik's and Sapatar's closest existing model is another
             # hybrid of attention and recurrent layers; the llama graph for
             # scale
             others = ((("livasun", livasun_spec),)
-                      if family in ("makezen", "fuvuvik") else ()) + (("llama_graph", llama_spec),)
+                      if family in ("makezen", "fuvuvik", "sapatar")
+                      else ()) + (("llama_graph", llama_spec),)
             for label, mk in ((family, mine),) + (() if solo else others):
                 pre, dec = engine_rates(mk(s, moe), device)
                 row[label] = {"prefill_tok_s": round(pre), "decode_tok_s": round(dec)}
@@ -1173,6 +1431,7 @@ def run(sizes: list[str], device: str, family: str = "vunitar",
             rates = {"vunitar": kernel_rates, "fusipel": fusipel_kernel_rates,
                      "livasun": livasun_kernel_rates,
                      "makezen": makezen_kernel_rates,
-                     "fuvuvik": fuvuvik_kernel_rates}[family]
+                     "fuvuvik": fuvuvik_kernel_rates,
+                     "sapatar": sapatar_kernel_rates}[family]
             for k in rates(s, device):
                 print(json.dumps({"kernel_bench": {"size": name, **k}}), flush=True)
