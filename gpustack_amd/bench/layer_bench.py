@@ -1369,7 +1369,7 @@ def sapatar_kernel_rates(s, device):
         y = torch.empty(T, nq, device=device)
         st = torch.zeros(nseq + 1, H, D, D, device=device)
         ext = torch.zeros(nseq + 1, H, D + 1, device=device)
-        b1 = torch.ones(H, device=device)
+        b1, rd = torch.ones(H, device=device), torch.empty(T, H, device=device)
         tab = ops.rope_table(ps, inv) if L > 1 else None
         N6 = W // 64
         st6 = torch.zeros(nseq + 1, N6, 64, 64, device=device)
@@ -1384,7 +1384,7 @@ def sapatar_kernel_rates(s, device):
             ("mlstm", nq * D, lambda: ops.memory_scan(
                 y, q, k, v, st, *view, q_scale=D ** -0.5,
                 gates=u[:, 4 * nq:], i_b=b1, f_b=b1, cap=15.0, extra=ext,
-                single=L == 1)),
+                rden=rd, single=L == 1)),
             ("wkv", W * 64, lambda: ops.memory_scan(
                 y6, r6, k6, v6, st6, *view, chan=z6, w0=w0, bonus=bo,
                 single=L == 1)),

@@ -241,10 +241,10 @@ class _MemoryMixer(nn.Module):
                         rg.state_slots, rg.pos32, single=rg.single, **kw)
         return y
 
-    def _norm(self, y, gate):
+    def _norm(self, y, gate, y_scale=None):
         g = torch.empty(y.shape, dtype=gate.dtype, device=y.device)
         ops.gated_group_norm(g, y, gate, self.norm, self.m.heads, self.eps,
-                             self.gate_mode)
+                             self.gate_mode, y_scale)
         return g
 
     def forward(self, h, *args, **kw):
@@ -322,10 +322,13 @@ class MlstmMixer(_MemoryMixer):
     def rows(self, h, meta, state, extra):
         m, n, g, i = self.m, self.nqk, self.col_g, self.col_i
         u = F.linear(h, self.in_w)
+        rden = torch.empty(h.shape[0], m.heads, dtype=torch.float32,
+                           device=h.device)
         y = self._scan(u[:, :n], u[:, n:2 * n], u[:, 2 * n:g], meta, state,
                        q_scale=m.state ** -0.5, gates=u[:, i:i + 2 * m.heads],
-                       i_b=self.i_b, f_b=self.f_b, cap=m.gate_cap, extra=extra)
-        return self._norm(y, u[:, g:i])
+                       i_b=self.i_b, f_b=self.f_b, cap=m.gate_cap, extra=extra,
+                       rden=rden)
+        return self._norm(y, u[:, g:i], rden)
 
 
 def build_scan_mixer(width: int, m: ScanMixerSpec, eps: float, dtype,

@@ -891,14 +891,17 @@ def state_scan(y, src, col_x: int, col_b: int, col_c: int, dt_src,
 
 
 def gated_group_norm(out, y, gate, w, groups: int, eps: float,
-                     gate_first) -> None:
+                     gate_first, y_scale=None) -> None:
     """gate_first: True / 1 = silu gate, then norm; False / 0 = norm, then
-    sigmoid gate; 2 = norm, then silu gate."""
+    sigmoid gate; 2 = norm, then silu gate. y_scale [T, groups] multiplies
+    the parts of y first."""
     k = _state_backend(y)
     if k is not None:
-        k.gated_group_norm(out, y, gate, w, groups, eps, int(gate_first))
+        k.gated_group_norm(out, y, gate, w, groups, eps, int(gate_first),
+                           y_scale)
     else:
-        torch_ref.gated_group_norm(out, y, gate, w, groups, eps, gate_first)
+        torch_ref.gated_group_norm(out, y, gate, w, groups, eps, gate_first,
+                                   y_scale)
 
 
 def route_topk(experts, weights, logits, correction, n_experts: int,
@@ -946,8 +949,8 @@ def rope_table(pos32, inv_freq):
 def memory_scan(y, q, k, v, state, seq_first, seq_rows, state_slots, pos32, *,
                 q_scale: float = 1.0, k_scale: float = 1.0, decay=None,
                 chan=None, w0=None, bonus=None, gates=None, i_b=None,
-                f_b=None, cap: float = 0.0, extra=None, inv_freq=None,
-                rot=None, single: bool = False) -> None:
+                f_b=None, cap: float = 0.0, extra=None, rden=None,
+                inv_freq=None, rot=None, single: bool = False) -> None:
     """Matrix memory over the state pool (torch_ref.memory_scan has the
     semantics). `single`: every sequence brings one row (a decode step).
     `rot`: the step's rope_table, shared by the layers of a prompt (None: the
@@ -955,12 +958,12 @@ def memory_scan(y, q, k, v, state, seq_first, seq_rows, state_slots, pos32, *,
     b = _state_backend(q)
     if b is not None:
         b.memory_scan(y, q, k, v, q_scale, k_scale, decay, chan, w0, bonus,
-                      rot, inv_freq, gates, i_b, f_b, cap, state, extra,
+                      rot, inv_freq, gates, i_b, f_b, cap, state, extra, rden,
                       seq_first, seq_rows, state_slots, pos32, single)
     else:
         torch_ref.memory_scan(y, q, k, v, state, seq_first, seq_rows,
                               state_slots, pos32, q_scale, k_scale, decay,
-                              chan, w0, bonus, gates, i_b, f_b, cap, extra,
+                              chan, w0, bonus, gates, i_b, f_b, cap, extra, rden,
                               inv_freq)
 
 

@@ -4,9 +4,9 @@
 //   CONST : S_t = a S + k v^T                 y = S_t^T q      a per head
 //   CHAN  : S_t = diag(w_t) S + k v^T         y = (S_(t-1) + diag(u) k v^T)^T q
 //           w_t = exp(-exp(z_t + w0)) per head and state row
-//   GATED : S_t = a_t S + b_t k v^T           y = S_t^T q / (max(|n_t . q|,
-//           exp(-m_t)) + 1e-6), n_t = a_t n + b_t k, with a_t = exp(f + m_(t-1)
-//           - m_t), b_t = exp(i - m_t), m_t = max(f + m_(t-1), i)
+//   GATED : S_t = a_t S + b_t k v^T           y = S_t^T q, to be divided by
+//           max(|n_t . q|, exp(-m_t)) + 1e-6, n_t = a_t n + b_t k, with a_t =
+//           exp(f + m_(t-1) - m_t), b_t = exp(i - m_t), m_t = max(f + m_(t-1), i)
 //
 // q and k may turn with the row's position (channel i with i + half) and carry
 // a constant factor. S lives in the sequence's slot of a state pool [slots, H,
@@ -16,11 +16,13 @@
 //
 //   rope_table       : cos / sin of every row's angles, once per step
 //   memory_gates     : GATED, prompts: a wave per (sequence, head) turns 64
-//                      rows' gates into (a, b) with a max-plus prefix scan,
-//                      walks n and leaves every row's denominator
+//                      rows' gates into (a, b) with a max-plus prefix scan
 //   memory_scan      : prompts. TPP neighbouring lanes share two value
 //                      channels, NR state rows each, in registers; rows are
-//                      staged through LDS and walked in order
+//                      staged through LDS and walked in order, the next
+//                      row's operands on their way while one is worked on.
+//                      GATED: one more workgroup per (sequence, head) walks n
+//                      as a state whose value is always 1
 //   memory_step      : single rows (decode): one pass over the state
 #include "common.h"
 
@@ -51,8 +53,9 @@ struct MemArgs {
   long ld_g;
   const float *i_b, *f_b;        // GATED: [H]
   float cap;
-  float* ab;                     // GATED, prompts: [T, H, 2]
-  float* rden;                   // GATED, prompts: [T, H] 1 / denominator
+  float* ab;                     // GATED, prompts: [T, H, 3] a, b, exp(-m)
+  float* rden;                   // GATED: [T, H] 1 / denominator, left to the
+                                 // reader of y
   float* state;                  // [nslots, H, N, P]
   float* extra;                  // GATED: [nslots, H, N + 1]
   const int* seq_first;
@@ -110,33 +113,34 @@ __global__ __launch_bounds__(64) void rope_table_kernel(
   }
 }
 
-// ---- GATED: gates, normaliser and denominators of a prompt ------------------
+// ---- GATED: the gates of a prompt ---------------------------------------------
 
-// NL: state rows per lane (N <= 64 NL)
-template <typename TS, int NL>
+template <typename TS>
 __global__ __launch_bounds__(64) void memory_gates_kernel(MemArgs p) {
   const int s = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const SeqView sv = view_of(p, s);
   if (!sv.ok) return;
-  const int H = p.H, N = p.N;
-  float* ex = p.extra + (sv.slot * H + h) * (N + 1);
-  float nv[NL];
-#pragma unroll
-  for (int j = 0; j < NL; ++j) {
-    const int e = lane + j * 64;
-    nv[j] = sv.has && e < N ? ex[e] : 0.f;
-  }
-  float m_in = sv.has ? ex[N] : 0.f;
+  const int H = p.H;
+  float* mp = p.extra + (sv.slot * H + h) * (p.N + 1) + p.N;
+  float m_in = sv.has ? *mp : 0.f;
   const float ib = p.i_b[h], fb = p.f_b[h];
+  float zi = 0.f, zf = 0.f;
+  auto fetch = [&](int c0) {
+    if (c0 + lane < sv.n) {
+      const TS* g = (const TS*)p.gates + (long)(sv.first + c0 + lane) * p.ld_g + h;
+      zi = ld(g);
+      zf = ld(g + H);
+    }
+  };
+  fetch(0);
   for (int c0 = 0; c0 < sv.n; c0 += 64) {
     const int rows = min(64, sv.n - c0);
-    const long t0 = sv.first + c0;
     float gi = -INFINITY, gf = 0.f;        // rows past the end keep m
     if (lane < rows) {
-      const TS* g = (const TS*)p.gates + (t0 + lane) * p.ld_g + h;
-      gi = capped(ld(g) + ib, p.cap);
-      gf = log_sigmoid_f(capped(ld(g + H) + fb, p.cap));
+      gi = capped(zi + ib, p.cap);
+      gf = log_sigmoid_f(capped(zf + fb, p.cap));
     }
+    fetch(c0 + 64);
     float F = gf, I = gi;                  // m -> max(F + m, I)
 #pragma unroll
     for (int d = 1; d < 64; d <<= 1) {
@@ -147,60 +151,17 @@ __global__ __launch_bounds__(64) void memory_gates_kernel(MemArgs p) {
       }
     }
     const float m = fmaxf(F + m_in, I);
-    float mp = __shfl_up(m, 1, WAVE_SIZE);
-    if (lane == 0) mp = m_in;
-    const float a = expf(gf + mp - m), b = expf(gi - m);
+    float before = __shfl_up(m, 1, WAVE_SIZE);
+    if (lane == 0) before = m_in;
     if (lane < rows) {
-      float* o = p.ab + ((t0 + lane) * H + h) * 2;
-      o[0] = a;
-      o[1] = b;
+      float* o = p.ab + ((long)(sv.first + c0 + lane) * H + h) * 3;
+      o[0] = expf(gf + before - m);
+      o[1] = expf(gi - m);
+      o[2] = expf(-m);
     }
-    float mine = 0.f;                      // n . q of row `lane`
-    for (int r0 = 0; r0 < rows; r0 += 8) {
-      float kv[8][NL], qv[8][NL], part[8];
-#pragma unroll
-      for (int r = 0; r < 8; ++r) {
-        const long t = t0 + min(r0 + r, rows - 1);
-        const TS* kr = (const TS*)p.k + t * p.ld_k + (long)h * N;
-        const TS* qr = (const TS*)p.q + t * p.ld_q + (long)h * N;
-#pragma unroll
-        for (int j = 0; j < NL; ++j) {
-          const int e = lane + j * 64;
-          kv[r][j] = e < N ? ld(kr + e) * p.k_scale : 0.f;
-          qv[r][j] = e < N ? ld(qr + e) * p.q_scale : 0.f;
-        }
-      }
-#pragma unroll
-      for (int r = 0; r < 8; ++r) {
-        const float ar = __shfl(a, (r0 + r) & 63, WAVE_SIZE);
-        const float br = __shfl(b, (r0 + r) & 63, WAVE_SIZE);
-        part[r] = 0.f;
-        if (r0 + r < rows) {
-#pragma unroll
-          for (int j = 0; j < NL; ++j) {
-            nv[j] = ar * nv[j] + br * kv[r][j];
-            part[r] += nv[j] * qv[r][j];
-          }
-        }
-      }
-#pragma unroll
-      for (int d = 32; d >= 1; d >>= 1)
-#pragma unroll
-        for (int r = 0; r < 8; ++r) part[r] += __shfl_xor(part[r], d, WAVE_SIZE);
-#pragma unroll
-      for (int r = 0; r < 8; ++r)
-        if (lane == r0 + r) mine = part[r];
-    }
-    if (lane < rows)
-      p.rden[(t0 + lane) * H + h] = 1.0f / (fmaxf(fabsf(mine), expf(-m)) + 1e-6f);
     m_in = __shfl(m, rows - 1, WAVE_SIZE);
   }
-#pragma unroll
-  for (int j = 0; j < NL; ++j) {
-    const int e = lane + j * 64;
-    if (e < N) ex[e] = nv[j];
-  }
-  if (lane == 0) ex[N] = m_in;
+  if (lane == 0) *mp = m_in;
 }
 
 // ---- prompts ------------------------------------------------------------------
@@ -218,7 +179,15 @@ constexpr int scan_rows(int mode, int nr, int tpp) {
   return ch;
 }
 
-// grid (nseq, H, ceil(P / channels per workgroup)); blockDim 64 .. 256
+// one row's operands of a lane
+template <int MODE, int NR>
+struct RowOps {
+  f32x4 k[NR / 4], q[NR / 4], w[MODE == CHAN_DECAY ? NR / 4 : 1];
+  float v[VC], a, b;
+};
+
+// grid (nseq, H, ceil(P / channels per workgroup)), GATED one more in z;
+// blockDim 64 .. 256
 template <typename TS, int MODE, int NR, int TPP>
 __global__ __launch_bounds__(256) void memory_scan_kernel(
     float* __restrict__ y, MemArgs p) {
@@ -231,16 +200,20 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(
   __shared__ __attribute__((aligned(16))) float qs[2][CH][ROW];
   __shared__ __attribute__((aligned(16))) float ws[2][CH][WROW];
   __shared__ __attribute__((aligned(16))) float vs[2][CH][PBM];
-  __shared__ float sc[2][CH][4];           // a, b, 1 / denominator, bonus
+  __shared__ float sc[2][CH][4];           // a, b, exp(-m), bonus
   const int s = blockIdx.x, h = blockIdx.y;
   const int tid = threadIdx.x, nthr = blockDim.x;
   const int PB = nthr / TPP * VC, p0 = blockIdx.z * PB;
   const int ns = tid % TPP, pl = (tid / TPP) * VC;
   const SeqView sv = view_of(p, s);
   if (!sv.ok) return;
-  const int H = p.H, N = p.N, P = p.P, half = p.half;
-  const int pc = p0 + pl;
-  float* sp = p.state + (sv.slot * H + h) * (long)N * P;
+  const int H = p.H, N = p.N, half = p.half;
+  // the normaliser: a state of one channel whose value is 1
+  const bool norm = MODE == GATED && blockIdx.z + 1 == gridDim.z;
+  const int P = norm ? 1 : p.P;
+  const int pc = norm ? pl : p0 + pl;
+  float* sp = norm ? p.extra + (sv.slot * H + h) * (long)(N + 1)
+                   : p.state + (sv.slot * H + h) * (long)N * P;
   float S[VC][NR];
 #pragma unroll
   for (int j = 0; j < NR; ++j) {
@@ -249,6 +222,8 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(
     for (int c = 0; c < VC; ++c)
       S[c][j] = sv.has && nn < N && pc + c < P ? sp[(long)nn * P + pc + c] : 0.f;
   }
+  if (norm)
+    for (int i = tid; i < 2 * CH * PBM; i += nthr) (&vs[0][0][0])[i] = 1.f;
   // state rows past N keep k = q = w = 0
   for (int i = tid; i < 2 * CH * ROW; i += nthr) {
     (&ks[0][0][0])[i] = 0.f;
@@ -320,7 +295,7 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(
           }
         }
       }
-      for (int i = tid; i < rows * (PB / 8); i += nthr) {
+      for (int i = tid; !norm && i < rows * (PB / 8); i += nthr) {
         const int r = i / (PB / 8), c = (i % (PB / 8)) * 8;
         u16x8 v8 = {0, 0, 0, 0, 0, 0, 0, 0};
         if (p0 + c < P)
@@ -350,7 +325,7 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(
           ws[buf][r][at(e)] = expf(-expf(
               ld((const TS*)p.chan + t * p.ld_c + (long)h * N + e) + w0[e]));
       }
-      for (int i = tid; i < rows * PB; i += nthr) {
+      for (int i = tid; !norm && i < rows * PB; i += nthr) {
         const int r = i / PB, c = i % PB;
         vs[buf][r][c] = p0 + c < P
             ? ld((const TS*)p.v + (t0 + r) * p.ld_v + (long)h * P + p0 + c) : 0.f;
@@ -358,10 +333,10 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(
     }
     if constexpr (MODE == GATED) {
       if (tid < rows) {
-        const long g = (t0 + tid) * H + h;
-        sc[buf][tid][0] = p.ab[g * 2];
-        sc[buf][tid][1] = p.ab[g * 2 + 1];
-        sc[buf][tid][2] = p.rden[g];
+        const float* g = p.ab + ((t0 + tid) * H + h) * 3;
+        sc[buf][tid][0] = g[0];
+        sc[buf][tid][1] = g[1];
+        sc[buf][tid][2] = g[2];
       }
     }
   };
@@ -390,50 +365,88 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(
     const float* kb = &ks[buf][0][ns * NS];
     const float* qb = &qs[buf][0][ns * NS];
     const float* wb = &ws[buf][0][MODE == CHAN_DECAY ? ns * NS : 0];
-    for (int r = 0; r < rows; ++r) {
-      const float* vr = &vs[buf][r][pl];
-      float v[VC], acc[VC];
+    auto fetch = [&](int r, RowOps<MODE, NR>& o) {
 #pragma unroll
-      for (int c = 0; c < VC; ++c) { v[c] = vr[c]; acc[c] = 0.f; }
-      const float a = MODE == GATED ? sc[buf][r][0] : a_const;
-      float bv[VC];
-#pragma unroll
-      for (int c = 0; c < VC; ++c)
-        bv[c] = MODE == GATED ? sc[buf][r][1] * v[c] : v[c];
-#pragma unroll
-      for (int j = 0; j < NR; j += 4) {
-        const f32x4 k4 = *reinterpret_cast<const f32x4*>(kb + r * ROW + j);
-        const f32x4 q4 = *reinterpret_cast<const f32x4*>(qb + r * ROW + j);
-        if constexpr (MODE == CHAN_DECAY) {
-          const f32x4 w4 = *reinterpret_cast<const f32x4*>(wb + r * ROW + j);
-#pragma unroll
-          for (int x = 0; x < 4; ++x)
-#pragma unroll
-            for (int c = 0; c < VC; ++c) {
-              acc[c] += S[c][j + x] * q4[x];
-              S[c][j + x] = w4[x] * S[c][j + x] + k4[x] * bv[c];
-            }
-        } else {
-#pragma unroll
-          for (int x = 0; x < 4; ++x)
-#pragma unroll
-            for (int c = 0; c < VC; ++c) {
-              S[c][j + x] = a * S[c][j + x] + k4[x] * bv[c];
-              acc[c] += S[c][j + x] * q4[x];
-            }
-        }
+      for (int j = 0; j < NR / 4; ++j) {
+        o.k[j] = *reinterpret_cast<const f32x4*>(kb + r * ROW + j * 4);
+        o.q[j] = *reinterpret_cast<const f32x4*>(qb + r * ROW + j * 4);
+        if constexpr (MODE == CHAN_DECAY)
+          o.w[j] = *reinterpret_cast<const f32x4*>(wb + r * ROW + j * 4);
       }
 #pragma unroll
-      for (int c = 0; c < VC; ++c) acc[c] = lanes_sum<TPP>(acc[c]);
-      if (ns == 0) {
-        float* yo = y + (long)(sv.first + c0 + r) * H * P + (long)h * P + pc;
+      for (int c = 0; c < VC; ++c) o.v[c] = vs[buf][r][pl + c];
+      o.a = MODE == GATED ? sc[buf][r][0] : a_const;
+      o.b = MODE == GATED ? sc[buf][r][1] : 1.f;
+    };
+    // a lane keeps the sums of one row in TPP and stores them together
+    float out[VC];
 #pragma unroll
-        for (int c = 0; c < VC; ++c) {
-          float o = acc[c];
-          if constexpr (MODE == CHAN_DECAY) o += v[c] * sc[buf][r][3];
-          if constexpr (MODE == GATED) o *= sc[buf][r][2];
-          if (pc + c < P) yo[c] = o;
+    for (int c = 0; c < VC; ++c) out[c] = 0.f;
+    auto work = [&](int r, const RowOps<MODE, NR>& o) {
+      float acc[VC], bv[VC];
+#pragma unroll
+      for (int c = 0; c < VC; ++c) {
+        acc[c] = 0.f;
+        bv[c] = MODE == GATED ? o.b * o.v[c] : o.v[c];
+      }
+#pragma unroll
+      for (int j = 0; j < NR / 4; ++j)
+#pragma unroll
+        for (int x = 0; x < 4; ++x)
+#pragma unroll
+          for (int c = 0; c < VC; ++c) {
+            float& st = S[c][j * 4 + x];
+            if constexpr (MODE == CHAN_DECAY) {
+              acc[c] += st * o.q[j][x];
+              st = o.w[j][x] * st + o.k[j][x] * bv[c];
+            } else {
+              st = o.a * st + o.k[j][x] * bv[c];
+              acc[c] += st * o.q[j][x];
+            }
+          }
+      const bool mine = (r & (TPP - 1)) == ns;
+#pragma unroll
+      for (int c = 0; c < VC; ++c) {
+        acc[c] = lanes_sum<TPP>(acc[c]);
+        out[c] = mine ? acc[c] : out[c];
+      }
+      if ((r & (TPP - 1)) == TPP - 1 || r == rows - 1) {
+        const int rf = (r & ~(TPP - 1)) + ns;
+        if (rf <= r) {
+          const long t = sv.first + c0 + rf;
+          if (norm) {
+            if (pc == 0)
+              p.rden[t * H + h] =
+                  1.0f / (fmaxf(fabsf(out[0]), sc[buf][rf][2]) + 1e-6f);
+          } else {
+            float* yo = y + t * H * P + (long)h * P + pc;
+#pragma unroll
+            for (int c = 0; c < VC; ++c) {
+              float o2 = out[c];
+              if constexpr (MODE == CHAN_DECAY)
+                o2 += vs[buf][rf][pl + c] * sc[buf][rf][3];
+              if (pc + c < P) yo[c] = o2;
+            }
+          }
         }
+      }
+    };
+    if constexpr (NR <= 16) {
+      RowOps<MODE, NR> o0, o1;
+      fetch(0, o0);
+      for (int r = 0; r < rows; r += 2) {
+        fetch(min(r + 1, CH - 1), o1);
+        work(r, o0);
+        if (r + 1 < rows) {
+          fetch(min(r + 2, CH - 1), o0);
+          work(r + 1, o1);
+        }
+      }
+    } else {
+      RowOps<MODE, NR> o0;
+      for (int r = 0; r < rows; ++r) {
+        fetch(r, o0);
+        work(r, o0);
       }
     }
   }
@@ -555,13 +568,13 @@ __global__ __launch_bounds__(256) void memory_step_kernel(
       *reinterpret_cast<f32x4*>(part + r0 * P + cg * 4) = acc;
     }
     __syncthreads();
-    const float rden = MODE == GATED
-        ? 1.0f / (fmaxf(fabsf(total), expf(-m)) + 1e-6f) : 1.f;
+    if (MODE == GATED && tid == 0)
+      p.rden[t * H + h] = 1.0f / (fmaxf(fabsf(total), expf(-m)) + 1e-6f);
     for (int e = tid; e < P; e += 256) {
       float o = MODE == CHAN_DECAY ? total * vs[e] : 0.f;
       const int nr = min(RP, N);
       for (int x = 0; x < nr; ++x) o += part[x * P + e];
-      y[t * H * P + (long)h * P + e] = MODE == GATED ? o * rden : o;
+      y[t * H * P + (long)h * P + e] = o;
     }
   }
 }
@@ -572,7 +585,8 @@ void scan_go(float* y, const MemArgs& p, int nseq, hipStream_t s) {
   const int waves = min(4, (p.P + per_wave - 1) / per_wave);
   const int pb = waves * per_wave;
   memory_scan_kernel<TS, MODE, NR, TPP>
-      <<<dim3(nseq, p.H, (p.P + pb - 1) / pb), waves * 64, 0, s>>>(y, p);
+      <<<dim3(nseq, p.H, (p.P + pb - 1) / pb + (MODE == GATED ? 1 : 0)),
+         waves * 64, 0, s>>>(y, p);
 }
 
 template <typename TS, int MODE>
@@ -599,13 +613,8 @@ int mem_run(float* y, const MemArgs& p, int nseq, int single, hipStream_t s) {
     memory_step_kernel<TS, MODE><<<dim3(nseq, p.H), 256, smem, s>>>(y, p);
     return 1;
   }
-  if constexpr (MODE == GATED) {
-    const dim3 grid(nseq, p.H);
-    if (p.N <= 64) memory_gates_kernel<TS, 1><<<grid, 64, 0, s>>>(p);
-    else if (p.N <= 128) memory_gates_kernel<TS, 2><<<grid, 64, 0, s>>>(p);
-    else if (p.N <= 256) memory_gates_kernel<TS, 4><<<grid, 64, 0, s>>>(p);
-    else memory_gates_kernel<TS, 8><<<grid, 64, 0, s>>>(p);
-  }
+  if constexpr (MODE == GATED)
+    memory_gates_kernel<TS><<<dim3(nseq, p.H), 64, 0, s>>>(p);
   return scan_pick<TS, MODE>(y, p, nseq, s);
 }
 
@@ -623,7 +632,7 @@ int mem_mode(float* y, const MemArgs& p, int mode, int nseq, int single,
 
 int memory_scan_max_state() { return 512; }
 
-// the caller needs gate workspaces (ab, rden) unless the step kernel runs
+// the caller needs the gates' workspace (ab) unless the step kernel runs
 int memory_scan_steps(int P, int single) {
   return single && P % 4 == 0 && P / 4 <= 256;
 }

@@ -14,7 +14,7 @@ void head_norm_store_launch(void*, void*, long, int, int, int, const float*, con
 void value_page_store_launch(const void*, long, int, void*, const long*, long, const int*, int, int, int, int, int, int, hipStream_t);
 void route_topk_launch(int*, float*, const float*, int, const float*, int, int, int, int, int, int, int, int, float, hipStream_t);
 int state_scan_launch(float*, const void*, long, int, int, int, const void*, long, int, int, int, int, int, int, const float*, const float*, const float*, const float*, float*, const int*, const int*, const int*, const int*, int, int, int, int, int, hipStream_t);
-void gated_group_norm_launch(void*, const float*, const void*, long, const float*, int, int, int, float, int, int, int, hipStream_t);
+void gated_group_norm_launch(void*, const float*, const float*, const void*, long, const float*, int, int, int, float, int, int, int, hipStream_t);
 int delta_scan_launch(float*, const void*, long, int, int, int, const void*, long, int, int, int, int, int, int, const float*, const float*, float*, const int*, const int*, const int*, const int*, int, int, int, int, int, hipStream_t);
 int delta_scan_max_state();
 int state_scan_max_state();
@@ -335,8 +335,8 @@ void memory_scan(Tensor y, Tensor q, Tensor k, Tensor v, double q_scale,
                  double k_scale, OptTensor decay, OptTensor chan, OptTensor w0,
                  OptTensor bonus, OptTensor rot, OptTensor inv_freq,
                  OptTensor gates, OptTensor i_b, OptTensor f_b, double cap,
-                 Tensor state, OptTensor extra, Tensor seq_first,
-                 Tensor seq_rows, Tensor state_slots, Tensor pos32,
+                 Tensor state, OptTensor extra, OptTensor rden,
+                 Tensor seq_first, Tensor seq_rows, Tensor state_slots, Tensor pos32,
                  bool single) {
   chk(y, "y", at::kFloat);
   chk(state, "state", at::kFloat);
@@ -389,10 +389,13 @@ void memory_scan(Tensor y, Tensor q, Tensor k, Tensor v, double q_scale,
     TORCH_CHECK(extra->dim() == 3 && extra->size(0) == state.size(0) &&
                 extra->size(1) == H && extra->size(2) == N + 1);
     ep = extra->data_ptr<float>();
+    TORCH_CHECK(rden.has_value(), "gates leave the denominators in rden");
+    chk(*rden, "rden", at::kFloat);
+    TORCH_CHECK(rden->dim() == 2 && rden->size(0) == T && rden->size(1) == H);
+    rdp = rden->data_ptr<float>();
     if (!steps) {
       ws = at::empty({(long)T, (long)H, 3L}, y.options());
       abp = ws.data_ptr<float>();
-      rdp = abp + (long)T * H * 2;
     }
   }
   if (inv_freq.has_value() && inv_freq->numel() > 0) {
@@ -426,7 +429,7 @@ void memory_scan(Tensor y, Tensor q, Tensor k, Tensor v, double q_scale,
 }
 
 void gated_group_norm(Tensor out, Tensor y, Tensor gate, Tensor w, long groups,
-                      double eps, long gate_first) {
+                      double eps, long gate_first, OptTensor y_scale) {
   chk(y, "y", at::kFloat);
   chk(w, "w", at::kFloat);
   const int out_bf = act_kind(out, "out");
@@ -436,7 +439,14 @@ void gated_group_norm(Tensor out, Tensor y, Tensor gate, Tensor w, long groups,
   const int T = y.size(0), C = y.size(1);
   TORCH_CHECK(groups >= 1 && C % groups == 0 && w.numel() == C);
   TORCH_CHECK(gate_first >= 0 && gate_first <= 2);
-  gated_group_norm_launch(out.data_ptr(), y.data_ptr<float>(), gate.data_ptr(),
+  const float* ys = nullptr;
+  if (y_scale.has_value()) {
+    chk(*y_scale, "y_scale", at::kFloat);
+    TORCH_CHECK(y_scale->dim() == 2 && y_scale->size(0) == T &&
+                y_scale->size(1) == groups);
+    ys = y_scale->data_ptr<float>();
+  }
+  gated_group_norm_launch(out.data_ptr(), y.data_ptr<float>(), ys, gate.data_ptr(),
                           gate.stride(0), w.data_ptr<float>(), T, C,
                           (int)groups, (float)eps, (int)gate_first, gate_bf,
                           out_bf, cur_stream(y));

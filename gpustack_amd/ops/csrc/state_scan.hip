@@ -409,20 +409,22 @@ DEVICE_INLINE float block_sum(float v, float* red) {
 
 // grid (T, groups): one workgroup per (row, part). gate_first 1: u = y *
 // silu(gate), out = u / rms(u) * w; 0: out = y / rms(y) * w * sigmoid(gate);
-// 2: out = y / rms(y) * w * silu(gate).
+// 2: out = y / rms(y) * w * silu(gate). ysc [T, groups] (or null) multiplies y
+// first.
 template <typename TG, typename TO>
 __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_kernel(
     TO* __restrict__ out, const float* __restrict__ y,
-    const TG* __restrict__ gate, long ld_gate, const float* __restrict__ w,
+    const float* __restrict__ ysc, const TG* __restrict__ gate, long ld_gate, const float* __restrict__ w,
     int C, int gs, float eps, int gate_first) {
   __shared__ float red[4];
   const long t = blockIdx.x;
   const int c0 = blockIdx.y * gs;
   const float* yr = y + t * C + c0;
   const TG* gr = gate + t * ld_gate + c0;
+  const float sc = ysc != nullptr ? ysc[t * gridDim.y + blockIdx.y] : 1.f;
   float ss = 0.f;
   for (int i = threadIdx.x; i < gs; i += ROW_THREADS) {
-    float u = yr[i];
+    float u = yr[i] * sc;
     if (gate_first == 1) u *= silu_f(ld(gr + i));
     ss += u * u;
   }
@@ -430,7 +432,7 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_kernel(
   const float inv = 1.0f / sqrtf(ss / (float)gs + eps);
   for (int i = threadIdx.x; i < gs; i += ROW_THREADS) {
     const float gv = ld(gr + i);
-    float u = yr[i];
+    float u = yr[i] * sc;
     if (gate_first == 1) u = u * silu_f(gv) * inv * w[c0 + i];
     else if (gate_first == 2) u = u * inv * w[c0 + i] * silu_f(gv);
     else u = u * inv * w[c0 + i] * sigmoid_f(gv);
@@ -444,13 +446,14 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_kernel(
 template <int NV>
 __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_vec_kernel(
     unsigned short* __restrict__ out, const float* __restrict__ y,
-    const unsigned short* __restrict__ gate, long ld_gate,
+    const float* __restrict__ ysc, const unsigned short* __restrict__ gate, long ld_gate,
     const float* __restrict__ w, int C, int gs, float eps, int gate_first) {
   __shared__ float red[4];
   const long t = blockIdx.x;
   const int c0 = blockIdx.y * gs;
   const float* yr = y + t * C + c0;
   const unsigned short* gr = gate + t * ld_gate + c0;
+  const float sc = ysc != nullptr ? ysc[t * gridDim.y + blockIdx.y] : 1.f;
   float u[NV][4], gv[NV][4];
   float ss = 0.f;
 #pragma unroll
@@ -462,7 +465,8 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_vec_kernel(
 #pragma unroll
       for (int k = 0; k < 4; ++k) {
         gv[j][k] = bf2f(g4[k]);
-        u[j][k] = gate_first == 1 ? yv[k] * silu_f(gv[j][k]) : yv[k];
+        u[j][k] = yv[k] * sc;
+        if (gate_first == 1) u[j][k] *= silu_f(gv[j][k]);
         ss += u[j][k] * u[j][k];
       }
     }
@@ -493,7 +497,7 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_vec_kernel(
 template <int LPG>
 __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_small_kernel(
     unsigned short* __restrict__ out, const float* __restrict__ y,
-    const unsigned short* __restrict__ gate, long ld_gate,
+    const float* __restrict__ ysc, const unsigned short* __restrict__ gate, long ld_gate,
     const float* __restrict__ w, int C, int gs, int groups, float eps,
     int gate_first) {
   constexpr int GPW = 64 / LPG;
@@ -508,10 +512,12 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_small_kernel(
   if (live) {
     const f32x4 yv = *reinterpret_cast<const f32x4*>(y + t * C + c0);
     const u16x4 g4 = *reinterpret_cast<const u16x4*>(gate + t * ld_gate + c0);
+    const float sc = ysc != nullptr ? ysc[t * groups + grp] : 1.f;
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
       gv[k] = bf2f(g4[k]);
-      u[k] = gate_first == 1 ? yv[k] * silu_f(gv[k]) : yv[k];
+      u[k] = yv[k] * sc;
+      if (gate_first == 1) u[k] *= silu_f(gv[k]);
       ss += u[k] * u[k];
     }
   }
@@ -625,7 +631,8 @@ int state_scan_launch(float* y, const void* src, long ld_src, int col_x,
   return scan_pick<float, float>(y, src, dt_src, p, nseq, s);
 }
 
-void gated_group_norm_launch(void* out, const float* y, const void* gate,
+void gated_group_norm_launch(void* out, const float* y, const float* ysc,
+                             const void* gate,
                              long ld_gate, const float* w, int T, int C,
                              int groups, float eps, int gate_first, int gate_bf,
                              int out_bf, hipStream_t s) {
@@ -640,7 +647,7 @@ void gated_group_norm_launch(void* out, const float* y, const void* gate,
     const dim3 sgrid(T, (groups + gpb - 1) / gpb);
 #define GGN(L)                                                               \
   gated_group_norm_small_kernel<L><<<sgrid, ROW_THREADS, 0, s>>>(            \
-      (unsigned short*)out, y, (const unsigned short*)gate, ld_gate, w, C,   \
+      (unsigned short*)out, y, ysc, (const unsigned short*)gate, ld_gate, w, C,   \
       gs, groups, eps, gate_first)
     switch (lpg) {
       case 1: GGN(1); break;
@@ -658,32 +665,32 @@ void gated_group_norm_launch(void* out, const float* y, const void* gate,
       gs <= 4096 && ((uintptr_t)gate % 8) == 0) {
     if (gs <= 1024)
       gated_group_norm_vec_kernel<1><<<grid, ROW_THREADS, 0, s>>>(
-          (unsigned short*)out, y, (const unsigned short*)gate, ld_gate, w, C,
+          (unsigned short*)out, y, ysc, (const unsigned short*)gate, ld_gate, w, C,
           gs, eps, gate_first);
     else
       gated_group_norm_vec_kernel<4><<<grid, ROW_THREADS, 0, s>>>(
-          (unsigned short*)out, y, (const unsigned short*)gate, ld_gate, w, C,
+          (unsigned short*)out, y, ysc, (const unsigned short*)gate, ld_gate, w, C,
           gs, eps, gate_first);
     return;
   }
   if (gate_bf) {
     if (out_bf)
       gated_group_norm_kernel<unsigned short, unsigned short>
-          <<<grid, ROW_THREADS, 0, s>>>((unsigned short*)out, y,
+          <<<grid, ROW_THREADS, 0, s>>>((unsigned short*)out, y, ysc,
                                         (const unsigned short*)gate, ld_gate, w,
                                         C, gs, eps, gate_first);
     else
       gated_group_norm_kernel<unsigned short, float><<<grid, ROW_THREADS, 0, s>>>(
-          (float*)out, y, (const unsigned short*)gate, ld_gate, w, C, gs, eps,
+          (float*)out, y, ysc, (const unsigned short*)gate, ld_gate, w, C, gs, eps,
           gate_first);
   } else {
     if (out_bf)
       gated_group_norm_kernel<float, unsigned short><<<grid, ROW_THREADS, 0, s>>>(
-          (unsigned short*)out, y, (const float*)gate, ld_gate, w, C, gs, eps,
+          (unsigned short*)out, y, ysc, (const float*)gate, ld_gate, w, C, gs, eps,
           gate_first);
     else
       gated_group_norm_kernel<float, float><<<grid, ROW_THREADS, 0, s>>>(
-          (float*)out, y, (const float*)gate, ld_gate, w, C, gs, eps,
+          (float*)out, y, ysc, (const float*)gate, ld_gate, w, C, gs, eps,
           gate_first);
   }
 }

@@ -776,12 +776,15 @@ def state_scan(y: torch.Tensor, src: torch.Tensor, col_x: int, col_b: int,
 
 def gated_group_norm(out: torch.Tensor, y: torch.Tensor, gate: torch.Tensor,
                      w: torch.Tensor, groups: int, eps: float,
-                     gate_first) -> None:
+                     gate_first, y_scale: torch.Tensor | None = None) -> None:
     """gate_first True (1): u = y * silu(gate), then RMS norm of each of
     `groups` equal parts of the row by its own root mean square, times w.
     False (0): RMS norm of y in parts, times w, times sigmoid(gate). 2: the
-    same with silu(gate) in place of the sigmoid. y fp32 [T, C]."""
+    same with silu(gate) in place of the sigmoid. y fp32 [T, C]; y_scale
+    [T, groups] multiplies the parts of y before anything else."""
     T, C = y.shape
+    if y_scale is not None:
+        y = (y.view(T, groups, C // groups) * y_scale[:, :, None]).view(T, C)
     mode = int(gate_first)
     g = gate.float()
     u = y * (g * torch.sigmoid(g)) if mode == 1 else y
@@ -970,6 +973,7 @@ def memory_scan(y: torch.Tensor, q: torch.Tensor, k: torch.Tensor,
                 i_b: torch.Tensor | None = None,
                 f_b: torch.Tensor | None = None, cap: float = 0.0,
                 extra: torch.Tensor | None = None,
+                rden: torch.Tensor | None = None,
                 inv_freq: torch.Tensor | None = None) -> None:
     """Matrix memory, per sequence and head over this step's rows in order,
     all in fp32; S [N, P] is read from state[slot] (zero when the first row
@@ -985,8 +989,9 @@ def memory_scan(y: torch.Tensor, q: torch.Tensor, k: torch.Tensor,
                     i = cap tanh((. + i_b) / cap); f = logsigmoid(cap
                     tanh((. + f_b) / cap)); m' = max(f + m, i);
                     a = exp(f + m - m'), b = exp(i - m');
-                    S <- a S + b k v^T;  n <- a n + b k;
-                    y = S^T q / (max(|n . q|, exp(-m')) + 1e-6)
+                    S <- a S + b k v^T;  n <- a n + b k;  y = S^T q;
+                    rden [T, H] takes 1 / (max(|n . q|, exp(-m')) + 1e-6),
+                    the factor y is still to be multiplied by
     y: [T, H * P] fp32."""
     H, N, P = state.shape[1:]
     T = q.shape[0]
@@ -1032,9 +1037,9 @@ def memory_scan(y: torch.Tensor, q: torch.Tensor, k: torch.Tensor,
                 m = new
                 S = a[:, None, None] * S + b[:, None, None] * kv
                 nv = a[:, None] * nv + b[:, None] * kf[t]
-                den = torch.maximum((nv * qf[t]).sum(-1).abs(),
-                                    torch.exp(-m)) + 1e-6
-                o = (S * qf[t][:, :, None]).sum(1) / den[:, None]
+                rden[t] = 1.0 / (torch.maximum(
+                    (nv * qf[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6)
+                o = (S * qf[t][:, :, None]).sum(1)
             else:
                 S = decay.float()[:, None, None] * S + kv
                 o = (S * qf[t][:, :, None]).sum(1)

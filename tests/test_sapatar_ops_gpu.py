@@ -65,27 +65,30 @@ def run_both(kind, H, N, P, dtype, news, hists, slots, single=False, seed=0):
                        torch.rand(7, H, 1, generator=g)], -1) \
         if kind == "gated" else None
     sf, sr, ss, rs, ps = ragged(news, hists, slots)
-    ref = torch.zeros(T, H * P)
+    ref, rd_r = torch.zeros(T, H * P), torch.zeros(T, H)
     st_r = state.clone()
     ex_r = extra.clone() if extra is not None else None
     q, k, v, gt = split(wide, H, N, P, kind)
     torch_ref.memory_scan(ref, q, k, v, st_r, sf, sr, ss, ps, extra=ex_r,
-                          **gt, **kw)
+                          rden=rd_r, **gt, **kw)
     wg, kg = wide.cuda(), to_gpu(kw)
     q, k, v, gt = split(wg, H, N, P, kind)
     st_g = state.cuda()
     ex_g = extra.cuda() if extra is not None else None
     got = torch.zeros(T, H * P, device="cuda")
+    rden = torch.zeros(T, H, device="cuda")
     psg = ps.cuda()
     if kind == "rot" and not single:
         kg["rot"] = ops.rope_table(psg, kg["inv_freq"])
     ops.memory_scan(got, q, k, v, st_g, sf.cuda(), sr.cuda(), ss.cuda(), psg,
-                    extra=ex_g, single=single, **gt, **kg)
+                    extra=ex_g, rden=rden, single=single, **gt, **kg)
     what = f"{kind} {H} {N} {P} {dtype}"
     close(got, ref, torch.float32, what, tol=5e-5)
     close(st_g, st_r, torch.float32, what + " state", tol=5e-5)
     if extra is not None:
         close(ex_g, ex_r, torch.float32, what + " extra", tol=5e-5)
+        # a sum close to zero loses its digits to its terms
+        close(1 / rden, 1 / rd_r, torch.float32, what + " den", tol=5e-5)
         # slots of nobody in the batch are untouched
     idle = [i for i in range(7) if i not in slots]
     assert torch.equal(st_g.cpu()[idle], state[idle])
