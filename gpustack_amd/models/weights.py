@@ -66,12 +66,10 @@ def _layered_tensor_plan(model):
         plan.append(("final.norm.b", model.final_norm_b, same))
     if not getattr(model, "tied_head", False):
         plan.append(("head", model.lm_head, same))
-    seen = set()
     for i, layer in enumerate(model.layers):
         p = f"l{i}."
-        if id(layer) in seen:
-            continue                    # runs with an earlier layer's weights
-        seen.add(id(layer))
+        if model.spec.layers[i].weights_of >= 0:
+            continue                    # runs with another layer's weights
         if hasattr(layer, "port1"):
             plan += _stream_layer_plan(p, layer)
             continue

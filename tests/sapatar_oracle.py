@@ -171,9 +171,10 @@ def capped(z, cap):
     return cap * torch.tanh(z / cap)
 
 
-def mlstm_recurrence(q, k, v, i, f):
+def mlstm_recurrence(q, k, v, i, f, floor=True):
     """One head: q, k [T, D], v [T, P]; i, f [T] log gates. The running
-    maximum m starts at 0."""
+    maximum m starts at 0. floor False: a planted mistake, no lower bound
+    under the denominator."""
     T, D = k.shape
     S = torch.zeros(D, v.shape[1], dtype=F64)
     n = torch.zeros(D, dtype=F64)
@@ -185,7 +186,10 @@ def mlstm_recurrence(q, k, v, i, f):
         S = a * S + b * k[t][:, None] * v[t][None, :]
         n = a * n + b * k[t]
         m = new
-        den = torch.maximum((n @ q[t]).abs(), torch.exp(-m)) + 1e-6
+        den = (n @ q[t]).abs()
+        if floor:
+            den = torch.maximum(den, torch.exp(-m))
+        den = den + 1e-6
         out[t] = (S.t() @ q[t]) / den
     return out
 
@@ -198,7 +202,8 @@ def mlstm_half(h, m, w, p, eps):
     f = log_sigmoid(capped(h @ W("f").t() + W("f.b"), cap))
     q = heads_of(q * D ** -0.5, H)
     k, v = heads_of(k, H), heads_of(v, H)
-    o = [rms_unit(mlstm_recurrence(q[a], k[a], v[a], i[:, a], f[:, a]), eps)
+    o = [rms_unit(mlstm_recurrence(q[a], k[a], v[a], i[:, a], f[:, a],
+                                  not m.get("no_floor")), eps)
          for a in range(H)]
     return (torch.cat(o, -1) * W("norm") * torch.sigmoid(g)) @ W("o").t()
 
