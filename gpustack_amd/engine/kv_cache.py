@@ -398,10 +398,15 @@ class KVCache:
             free_bytes = max(0, free_bytes - (cfg.max_num_seqs + 1)
                              * spec.state_bytes_per_slot(esize))
             planes = KVCache.latent_planes(cfg)
-            per_block = max(1, cfg.block_size * esize * sum(
+            per_block = cfg.block_size * esize * sum(
                 w[1] * planes if w[0] == "latent" else
                 0 if w[0] in ("state", "shared") else w[1] * (w[2] + w[3])
-                for w in spec.kv_pool_widths()))
+                for w in spec.kv_pool_widths())
+            if per_block == 0:
+                # nothing is kept per token: blocks are bookkeeping only, as
+                # many as all admissible sequences can name
+                return cfg.max_num_seqs * -(-cfg.max_model_len
+                                            // cfg.block_size) + 1
         elif spec.kv_lora_rank:
             per_block = (nl * cfg.block_size
                          * (spec.kv_lora_rank + spec.qk_rope_head_dim)

@@ -618,6 +618,11 @@ def test_a_stack_without_attention(tmp_path):
     layers = [oracle.wkv_layer(), oracle.retention_layer()]
     steps = [[("a", 12)], [("a", 2)]] + [[("a", 1)]] * 6
     assert _one(tmp_path, layers, n=20, steps=steps) < TOL
+    # blocks without bytes are counted by what sequences can name, however
+    # much memory there is
+    eng = make_engine(str(tmp_path))
+    n = type(eng.runner.kv).compute_num_blocks(eng.cfg, 1 << 40)
+    assert n == 4 * (4096 // eng.cfg.block_size) + 1
 
 
 def test_bf16_engine_is_close(model):
